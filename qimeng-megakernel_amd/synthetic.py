@@ -23,6 +23,7 @@ import torch
 
 from .decode_schedule.globs import Globals
 from .decode_schedule.model_config import DecodeShape, LlamaConfig
+from .decode_schedule_hybrid.model_config import HybridShape, LayerShape
 
 BARRIER_ROWS = 10          # the reference's allocation
 XCD_COUNTER_ROWS = 54      # rows 10..53 hold the per-XCD sub-counters of the all-to-all edges
@@ -296,3 +297,84 @@ def build_moe_globals(weights: dict[str, torch.Tensor], shape: Any, kv_capacity:
     )
     g.embed_tokens = on_device["embed_tokens"]
     return g
+
+
+def hybrid_shape(pattern: str, *, width: int, vocab: int, streams: int, eps: float = 1e-5, ff: dict[str, int] | None = None, heads: int = 16, dim: int = 128,
+                 rot_dim: int = 64, v_dim: int = 128, rank: int = 512, window: int = 1024, rope_base: float = 10000.0, scale: float | None = None,
+                 lru_width: int = 2560, blocks: int = 10, taps: int = 4, wkv_heads: int = 32, wkv_dim: int = 64, wkv_rank: int = 64) -> HybridShape:
+    """A hybrid shape from a string of layers: ``r`` gated recurrence, ``a`` latent attention, ``w`` wkv; ``ff`` gives the
+    feed-forward size per letter (absent: none)."""
+    ff = ff or {}
+    kinds = {
+        "r": dict(type="rglru", lru_width=lru_width, blocks=blocks, taps=taps),
+        "a": dict(type="latent_attention", heads=heads, dim=dim, rot_dim=rot_dim, v_dim=v_dim, rank=rank, window=window, rope_base=rope_base,
+                  scale=(dim + rot_dim) ** -0.5 if scale is None else scale),
+        "w": dict(type="wkv", heads=wkv_heads, dim=wkv_dim, rank=wkv_rank),
+    }
+    return HybridShape(layers=tuple(LayerShape(ff=ff.get(c, 0), **kinds[c]) for c in pattern), width=width, vocab=vocab, streams=streams, eps=eps)
+
+
+#: about the parameters of the Llama-3.2-1B shape (width, feed-forward and vocabulary are its own)
+LUSUPEL_1B = hybrid_shape("raaw" * 4, width=2048, vocab=128256, streams=4, ff={"a": 8192, "r": 8192})
+#: about the parameters of the Qwen3-1.7B shape
+LUSUPEL_2B = hybrid_shape("raaw" * 7, width=2048, vocab=151936, streams=4, ff={"a": 6144, "r": 6144, "w": 6144}, window=2048)
+
+
+def random_hybrid_weights(shape: HybridShape, seed: int, device: torch.device | str = "cpu") -> dict[str, torch.Tensor]:
+    """Seeded random-init tensors of a hybrid decoder by checkpoint name, bf16.
+
+    Projections ~N(0, 1/fan-in) (embedding and head N(0, 1) and 1/fan-in), norm weights near one, the recurrence's decays
+    between slow and fast, the hyper-connections near a residual sum (a diagonal near one with small exchanges between the
+    streams).  Drawn on ``device``'s generator; on "cpu" a seed names the same model on every machine."""
+    from .decode_schedule_hybrid.weights import tensor_shapes
+
+    device = torch.device(device)
+    gen = torch.Generator(device=device)
+    gen.manual_seed(seed)
+    S = shape.streams
+
+    def normal(size: tuple[int, ...], scale: float = 1.0, mean: float = 0.0) -> torch.Tensor:
+        return mean + scale * torch.randn(*size, generator=gen, dtype=torch.float32, device=device)
+
+    def uniform(size: tuple[int, ...], low: float, high: float) -> torch.Tensor:
+        return low + (high - low) * torch.rand(*size, generator=gen, dtype=torch.float32, device=device)
+
+    out: dict[str, torch.Tensor] = {}
+    for name, size in tensor_shapes(shape).items():
+        part = name.split(".", 1)[-1] if name.startswith("l") else name
+        if name == "embed":
+            t = normal(size)
+        elif part.endswith("norm") or part in ("norm1", "norm2"):
+            t = normal(size, 0.1, 1.0)
+        elif part.startswith("hc"):
+            if part.endswith(".mix"):
+                t = torch.eye(S, device=device) + normal(size, 0.2 / S)
+            else:
+                t = normal(size, 0.3, 1.0 / S if part.endswith(".in") else 1.0)
+        elif part == "mix.lam":
+            t = uniform(size, -6.0, -2.0)          # decays of 1 - softplus(lam) x 8 x gate
+        elif part.startswith("mix.mu."):
+            t = uniform(size, 0.0, 1.0)
+        elif part == "mix.w0":
+            t = uniform(size, -6.0, 0.0)
+        elif part == "mix.u":
+            t = normal(size, 0.5)
+        elif part == "mix.conv":
+            t = normal(size, size[-1] ** -0.5)
+        elif part.endswith(".b"):
+            t = normal(size, 0.1)
+        else:
+            t = normal(size, size[-1] ** -0.5)
+        out[name] = t.to(torch.bfloat16)
+    return out
+
+
+def build_synthetic_hybrid_globals(shape: HybridShape, *, seed: int = 0, max_positions: int = 1032, slots: int = 1, portion_rows: int = 2048,
+                                   dtype: torch.dtype = torch.bfloat16, device: torch.device | str = "cuda") -> Any:
+    """Convenience: weights of ``seed`` drawn on ``device``, states and buffers of the hybrid route."""
+    from .decode_schedule_hybrid import HybridConfig, weights
+    from .decode_schedule_hybrid.globs import build_globals as build_hybrid
+
+    HybridConfig.set_shape(shape)
+    packed = weights.pack(shape, random_hybrid_weights(shape, seed, device), device)
+    return build_hybrid(shape, packed, dtype=dtype, slots=slots, max_positions=max_positions, portion_rows=portion_rows)
