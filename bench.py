@@ -37,6 +37,7 @@ ROOT = Path(__file__).resolve().parent
 sys.path.insert(0, str(ROOT))
 
 HBM_PEAK_GBPS = 8000.0
+MFMA_PEAK_FLOPS = 2.5e15   # dense bf16
 # HBM bytes one launch moves, from the two rocprofv3 --pmc runs (FETCH_SIZE, WRITE_SIZE; each scaled by
 # what the same counter reads for a 1 GiB copy) summarised in profiles/decode_megakernel_llama1b_hbm_counters.txt:
 # 1.0080 x the algorithmic bytes over the launches this file times by default with `--steps 20` (contexts 1012..1031);
@@ -499,6 +500,130 @@ def moe_decode_rows(args, shape, name: str, globs, kv_capacity: int, new_tokens:
     }
 
 
+HYBRID_PEER = {"lusupel-1b": "llama-3.2-1b", "lusupel-2b": "qwen3-1.7b"}   # the closest dense model at equal size
+
+
+def hybrid_decode(args) -> dict:
+    """Greedy decode and prefill of a hybrid (Lusupel) shape, beside the closest dense shape of about its size on the
+    same GPU: that one's decode through its own kernel, and its prefill, which is its decode kernel once per position."""
+    import torch
+
+    from qimeng_megakernel_amd import decode, decode_hybrid, registry, synthetic
+    from qimeng_megakernel_amd.decode_schedule import mk_kernel as dense_kernel
+    from qimeng_megakernel_amd.decode_schedule.model_config import LlamaConfig
+    from qimeng_megakernel_amd.decode_schedule_hybrid import mk_kernel
+    from qimeng_megakernel_amd.decode_schedule_hybrid.state import RequestTable
+
+    device = torch.device("cuda:0")
+    torch.cuda.set_device(device)
+    shape, peer_name = registry.shape_of(args.model), HYBRID_PEER[args.model]
+    lengths = [int(x) for x in args.prefill_lengths.split(",") if x.strip()]
+    new_tokens = max(args.new_tokens, args.steps + 1)
+    timed = min(args.steps, new_tokens - 1)
+    capacity = max([args.prompt_len + new_tokens] + lengths)
+    globs = synthetic.build_synthetic_hybrid_globals(shape, seed=args.seed, max_positions=capacity, portion_rows=4096, device=device)
+    mk = mk_kernel.get_mk()
+    gen = torch.Generator().manual_seed(args.seed + 1_000_003)
+    prompt = torch.randint(0, shape.vocab, (args.prompt_len,), generator=gen, dtype=torch.long)
+    if args.copy_calibration:
+        copy_calibration(device)
+    if args.warmup > 0:
+        decode_hybrid.decode(globs, prompt, min(args.warmup + 1, new_tokens), mk=mk, decode_time=False)
+    out = decode_hybrid.decode(globs, prompt, new_tokens, mk=mk, timed_steps=timed)
+    t, tokens = out["timing"], out["new_tokens"].tolist()
+    graph_tok_s = None
+    if not args.no_graph_run:
+        g_out = decode_hybrid.decode(globs, prompt, new_tokens, mk=mk, timed_steps=timed, use_graph=True)
+        if g_out["new_tokens"].tolist() != tokens:
+            raise SystemExit("bench.py: the graph replay produced different tokens than the launch loop")
+        graph_tok_s = g_out["timing"]["effective_tok_s_gpu"]
+
+    table, prefill = RequestTable(globs), {}
+    for n in lengths:
+        ids = torch.randint(0, shape.vocab, (n,), generator=gen, dtype=torch.long).to(device)
+        best = float("inf")
+        for it in range(4):
+            request = table.open("prefill")
+            a, b = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
+            a.record()
+            decode_hybrid.run_tokens(globs, mk, request, ids, [n - 1])
+            b.record()
+            torch.cuda.synchronize(device)
+            table.close("prefill")
+            if it:
+                best = min(best, a.elapsed_time(b) / 1e3)
+        flops = shape.prefill_flops(n)
+        prefill[str(n)] = {"tok_s": n / best, "ms": best * 1e3, "tflops": flops / best / 1e12, "mfma_frac": flops / best / MFMA_PEAK_FLOPS}
+    del globs
+    torch.cuda.empty_cache()
+
+    peer = registry.shape_of(peer_name)
+    LlamaConfig.set_shape(peer)
+    peer_globs = synthetic.build_globals(synthetic.random_weights(peer, args.seed, args.prompt_len + new_tokens), peer, args.prompt_len + new_tokens, device)
+    peer_mk = dense_kernel.get_mk()
+    decode.decode(peer_globs, prompt % peer.vocab_size, 17, mk=peer_mk, decode_time=False)
+    p = decode.decode(peer_globs, prompt % peer.vocab_size, new_tokens, mk=peer_mk, device_sampling=True, timed_steps=timed)["timing"]
+    return {
+        "metric": "kernel_tok_s", "value": t["kernel_tok_s"], "unit": "tok/s", "n_gpus": 1, "steps": timed, "warmup": args.warmup,
+        "ms_per_step": t["kernel_ms_per_step"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+        "config": {"workload": f"{args.model} shape, batch-1 greedy decode, {args.prompt_len}-token prompt, {new_tokens} new tokens; timed: the last {timed} "
+                               f"decode steps (contexts {t['first_timed_context']}..{t['last_timed_context']}), seeded random-init bf16 weights; prefill of "
+                               f"random prompts in portions of up to 4096 tokens",
+                   "layers": len(shape.layers), "mixers": "".join({"rglru": "r", "latent_attention": "a", "wkv": "w"}[l.type] for l in shape.layers),
+                   "hidden": shape.width, "streams": shape.streams, "vocab": shape.vocab, "weight_bytes": shape.weight_bytes_per_token(), "batch": 1,
+                   "seed": args.seed},
+        "tok_s": t["effective_tok_s_wall"], "tok_s_gpu": t["effective_tok_s_gpu"], "kernel_tok_s": t["kernel_tok_s"], "tok_s_gpu_graph": graph_tok_s,
+        "roofline": {"bound": "hbm", "achieved": t["achieved_GBps"], "peak": HBM_PEAK_GBPS, "unit": "GB/s", "frac": t["achieved_GBps"] / HBM_PEAK_GBPS,
+                     "bytes_per_launch_avg": t["algorithmic_bytes"] / max(timed, 1), "kernel": "decode_megakernel_hybrid"},
+        "prefill": prefill,
+        "closest_model": {"model": peer_name, "weight_bytes": peer.weight_bytes_per_token(), "kernel_tok_s": p["kernel_tok_s"],
+                          "ms_per_step": p["kernel_ms_per_step"], "roofline_frac": p["achieved_GBps"] / HBM_PEAK_GBPS,
+                          "prefill_tok_s": p["kernel_tok_s"], "prefill": "its decode kernel once per prompt position"},
+    }
+
+
+def hybrid_phase_table(name: str, context: int = 1000) -> dict:
+    """One decode step of a hybrid shape with timeline records: per opcode the mean time from the end of the stage before
+    to the end of the stage, and the stage's weight bytes over it."""
+    import numpy as np
+    import torch
+
+    from qimeng_megakernel_amd import decode_hybrid, registry, synthetic
+    from qimeng_megakernel_amd.decode_schedule_hybrid import mk_kernel
+    from qimeng_megakernel_amd.decode_schedule_hybrid.instructions import scheduler
+    from qimeng_megakernel_amd.decode_schedule_hybrid.state import RequestTable
+
+    shape = registry.shape_of(name)
+    g = synthetic.build_synthetic_hybrid_globals(shape, max_positions=context + 8, device="cuda:0")
+    mk = mk_kernel.get_mk()
+    request = RequestTable(g).open(0)
+    ids = torch.randint(0, shape.vocab, (context - 1,), generator=torch.Generator().manual_seed(1))
+    decode_hybrid.run_tokens(g, mk, request, ids)
+    for _ in range(3):
+        decode_hybrid.run_tokens(g, mk, request, [5])
+    mk.timeline = torch.zeros(*g.instructions.shape[:2], 8, dtype=torch.int64, device="cuda:0")
+    decode_hybrid.run_tokens(g, mk, request, [5])
+    mk.check()
+    t = mk.timeline.cpu().numpy().astype(np.int64)
+    stages, queues = scheduler.HybridScheduler(shape, max_positions=g.max_positions).stages(), int(g.instructions.shape[0])
+    ends, kinds, index = [], [], [0] * queues
+    for stage in stages:
+        last = 0
+        for k, _ in enumerate(stage):
+            q = k % queues
+            last = max(last, int(t[q, index[q], 2]))
+            index[q] += 1
+        ins = stage[0]
+        layer = shape.layers[ins.layer]
+        kinds.append(type(ins).__name__ + {0: "", 1: "_down"}.get(ins.sub if ins.opcode() == 7 else 0, "") + ("" if ins.opcode() == 9 else ":" + layer.type))
+        ends.append(last)
+    start = int(t[..., 0][t[..., 0] > 0].min())
+    rows: dict = {}
+    for k, kind in enumerate(kinds):
+        rows.setdefault(kind, []).append((ends[k] - (ends[k - 1] if k else start)) / 100.0)
+    return {"total_us": (ends[-1] - start) / 100.0, "stages": {k: {"count": len(v), "mean_us": sum(v) / len(v), "sum_us": sum(v)} for k, v in rows.items()}}
+
+
 def cpu_baseline_batch(shape, weights, prompts, n_steps: int, cores: int, shape_name: str) -> dict:
     """The fused batch oracle on the host cores: ``n_steps`` steps of the same rows from position 0."""
     import torch
@@ -543,11 +668,13 @@ def main() -> None:
     ap.add_argument("--length-bench-iters", type=int, default=5)
     ap.add_argument("--cpu-steps", type=int, default=16)
     ap.add_argument("--no-cpu-baseline", action="store_true")
-    ap.add_argument("--model", choices=("llama-3.2-1b", "qwen3-1.7b", "qwen1.5-moe-a2.7b", "qwen3-30b-a3b"), default="llama-3.2-1b",
+    ap.add_argument("--model", choices=("llama-3.2-1b", "qwen3-1.7b", "qwen1.5-moe-a2.7b", "qwen3-30b-a3b", "lusupel-1b", "lusupel-2b"), default="llama-3.2-1b",
                     help="layer geometry: the headline Llama-3.2-1B shape, the Qwen3-1.7B shape with the Qwen3 op set "
                          "(28 layers, per-head QK RMSNorm, tied LM head), the Qwen1.5-MoE-A2.7B shape with the MoE op set "
                          "(24 layers, 60 experts of 1408 with top-4 routing, shared expert of 5632), or the Qwen3-30B-A3B shape "
-                         "(48 layers, 128 experts of 768 with renormalised top-8 routing, 32/4 heads of 128; 512 new tokens)")
+                         "(48 layers, 128 experts of 768 with renormalised top-8 routing, 32/4 heads of 128; 512 new tokens), "
+                         "or a hybrid (Lusupel) shape: decode and prefill, beside the dense shape of about its size")
+    ap.add_argument("--prefill-lengths", default="512,2048,4096", help="hybrid shapes: prompt lengths whose prefill is timed")
     ap.add_argument("--host-sampling", action="store_true",
                     help="argmax and embedding lookup on the host between launches, as the reference's loop does "
                          "(default: inside the kernel)")
@@ -576,17 +703,25 @@ def main() -> None:
 
     import torch
 
-    from __graft_entry__ import LIBRARY, build_library, load_package
+    from __graft_entry__ import HYBRID_LIBRARY, LIBRARY, build_library, load_package
 
     if not torch.cuda.is_available():
         raise SystemExit("bench.py needs a GPU")
     if not LIBRARY.is_file():
         build_library()
+    if args.model in HYBRID_PEER and not HYBRID_LIBRARY.is_file():
+        build_library(HYBRID_LIBRARY)
     load_package()
     from qimeng_megakernel_amd import decode, synthetic
     from qimeng_megakernel_amd.decode_schedule import mk_kernel
     from qimeng_megakernel_amd.decode_schedule.model_config import LLAMA_3_2_1B, QWEN3_1_7B, LlamaConfig
 
+    if args.model in HYBRID_PEER:
+        if args.batch != 1:
+            raise SystemExit("bench.py: the hybrid route decodes one request at a time")
+        print(json.dumps({"metric": "stage_us", "unit": "us", "config": {"workload": f"{args.model} shape, one decode step at context 1000"},
+                          **hybrid_phase_table(args.model)} if args.phase_table else hybrid_decode(args)))
+        return
     if args.phase_table:
         res = phase_table()
         print(json.dumps({"metric": "phase_GBps", "unit": "GB/s", "n_gpus": 1, "higher_is_better": True, "dtype": "bf16", "data": "synthetic",

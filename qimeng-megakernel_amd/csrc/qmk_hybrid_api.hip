@@ -7,6 +7,7 @@
 
 #include <algorithm>
 #include <mutex>
+#include <type_traits>
 
 #include "qmk_hybrid_ops.h"
 #include "qmk_hybrid_prefill.h"
@@ -19,24 +20,42 @@ constexpr int kMaxDevices = 16;
 constexpr int kMaxQueues = 1024;
 __device__ int32_t g_status[kStatusWords];
 
+// The launch's parameters as one instruction sees them: read from the kernel-argument segment through a pointer the
+// compiler cannot look behind, so that an op loads what it needs of them and keeps nothing across the instruction loop
+// (held in scalar registers for the whole kernel they are parked in vector lanes, one move per use).
+static_assert(std::is_trivially_copyable<DecodeParams>::value && std::is_standard_layout<DecodeParams>::value, "copied byte for byte into the segment");
+__device__ __forceinline__ const DecodeParams& params_of_this_instruction() {
+  auto args = __builtin_amdgcn_kernarg_segment_ptr();
+  asm volatile("" : "+s"(args));
+  return *(const DecodeParams*)args;   // the only kernel argument: offset 0 of the segment
+}
+
 template <class T>
-__global__ __launch_bounds__(kThreads, 1) void decode_megakernel_hybrid(const DecodeParams p) {
+__global__ __launch_bounds__(kThreads, 1) void decode_megakernel_hybrid(const DecodeParams p_launch) {
+  const DecodeParams& p_loop = p_launch;
   __shared__ __align__(16) Smem s;
   if (threadIdx.x == 0) {
     s.best_val = -INFINITY;
     s.best_idx = 0x7fffffff;
   }
-  const int32_t* queue = p.instructions + static_cast<size_t>(blockIdx.x) * p.num_insts * kInstWords;
+  const int num_insts = p_loop.num_insts;
+  const int32_t* queue = p_loop.instructions + static_cast<size_t>(blockIdx.x) * num_insts * kInstWords;
   bool ok = true;
-  int32_t word = (threadIdx.x < kInstWords && p.num_insts > 0) ? queue[threadIdx.x] : 0;
-  for (int i = 0; i < p.num_insts && ok; ++i) {
+  // The words of instruction i + 2 are asked for while instruction i runs.
+  int32_t word = (threadIdx.x < kInstWords && num_insts > 0) ? queue[threadIdx.x] : 0;
+  int32_t word1 = (threadIdx.x < kInstWords && num_insts > 1) ? queue[kInstWords + threadIdx.x] : 0;
+  for (int i = 0; i < num_insts && ok; ++i) {
     if (threadIdx.x < kInstWords) {
       s.inst[threadIdx.x] = word;
-      word = (i + 1 < p.num_insts) ? queue[(i + 1) * kInstWords + threadIdx.x] : 0;
+      if (threadIdx.x == 1) s.next_layer = word1;
+      word = word1;
+      word1 = (i + 2 < num_insts) ? queue[(i + 2) * kInstWords + threadIdx.x] : 0;
     }
     __syncthreads();
+    const DecodeParams& p = params_of_this_instruction();
     auto operand = [&](int w) { return __builtin_amdgcn_readfirstlane(s.inst[w]); };
-    const Op o{i, operand(0), operand(1), operand(2), operand(3), operand(4), operand(5), operand(6), operand(7), operand(8)};
+    const int next_layer = __builtin_amdgcn_readfirstlane(s.next_layer);
+    const Op o{next_layer >= 0 && next_layer < p.num_layers ? next_layer : 0, i, operand(0), operand(1), operand(2), operand(3), operand(4), operand(5), operand(6), operand(7), operand(8)};
     unsigned long long t_start = 0;
     if (p.timeline != nullptr && threadIdx.x == 0) t_start = s.t_wait = wall_clock64();
     if (o.opcode != OP_NOOP && (o.layer < 0 || o.layer >= p.num_layers || o.wait_stage >= 4 * p.groups || o.arrive_stage >= 4 * p.groups)) {
@@ -44,15 +63,15 @@ __global__ __launch_bounds__(kThreads, 1) void decode_megakernel_hybrid(const De
     } else {
       switch (o.opcode) {
         case OP_NOOP: break;
-        case OP_IN_PROJECT: ok = op_in_project(p, s, o); break;
-        case OP_LRU_STEP: ok = op_lru_step(p, s, o); break;
-        case OP_LATENT_ABSORB: ok = op_latent_absorb<T>(p, s, o); break;
+        case OP_IN_PROJECT:
+        case OP_LRU_STEP:
+        case OP_LATENT_ABSORB:
+        case OP_LATENT_VALUE:
+        case OP_WKV_STEP:
+        case OP_OUT_PROJECT:
+        case OP_UP_GATE:
+        case OP_LM_HEAD: ok = op_rows<T>(p, s, o); break;
         case OP_LATENT_ATTEND: ok = op_latent_attend<T>(p, s, o); break;
-        case OP_LATENT_VALUE: ok = op_latent_value(p, s, o); break;
-        case OP_WKV_STEP: ok = op_wkv_step(p, s, o); break;
-        case OP_OUT_PROJECT: ok = op_out_project(p, s, o); break;
-        case OP_UP_GATE: ok = op_up_gate(p, s, o); break;
-        case OP_LM_HEAD: ok = op_lm_head(p, s, o); break;
         default:
           if (threadIdx.x == 0) report_error(counters_of(p), QMK_DEV_BAD_OPCODE, i, o.opcode, 0);
           ok = false;
@@ -65,10 +84,12 @@ __global__ __launch_bounds__(kThreads, 1) void decode_megakernel_hybrid(const De
       rec[1] = s.t_wait;
       rec[2] = wall_clock64();
       rec[3] = static_cast<uint64_t>(o.opcode) | (static_cast<uint64_t>(static_cast<uint32_t>(o.layer)) << 8);
+      for (int k = 0; k < 4; ++k) rec[4 + k] = s.stamps[k];
     }
     __syncthreads();
   }
   if (!ok) return;
+  const DecodeParams& p = params_of_this_instruction();
 
   // Retire: the last workgroup to arrive owns the counters alone, clears them and picks the token among the
   // workgroups' candidates (largest logit, smallest row among equals).

@@ -184,8 +184,10 @@ __global__ __launch_bounds__(kPfThreads) void gemm(const GemmArgs g) {
   constexpr int kRowA = kBK / kUnitA, kRowW = kBK / kUnitW;                // units of a row
   constexpr int kLoadsA = BM * kRowA / kPfThreads, kLoadsW = BN * kRowW / kPfThreads;
   constexpr int kTm = BM / 2 / 16, kTn = BN / 2 / 16;
-  __shared__ v4u la[2][BM * kRowA];
-  __shared__ v4u lw[2][BN * kRowW];
+  constexpr int kTileUnits = 2 * (BM * kRowA + BN * kRowW), kOutUnits = BM * BN / 4;
+  __shared__ v4u lds[kTileUnits > kOutUnits ? kTileUnits : kOutUnits];
+  v4u(*la)[BM * kRowA] = reinterpret_cast<v4u(*)[BM * kRowA]>(lds);
+  v4u(*lw)[BN * kRowW] = reinterpret_cast<v4u(*)[BN * kRowW]>(lds + 2 * BM * kRowA);
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, wm = wave & 1, wn = wave >> 1;
   const int group = blockIdx.z;
   const int N = group == g.groups - 1 ? g.last_n : g.N;
@@ -250,16 +252,21 @@ __global__ __launch_bounds__(kPfThreads) void gemm(const GemmArgs g) {
     if (s + 1 < steps) stash(buf ^ 1);
     __syncthreads();
   }
+  // Through LDS (a wave's own 64 x 64 part, quads of a row exchanged by its number): a lane's accumulators are then read
+  // back in a loop, and sixteen lanes write 64 neighbouring outputs of one token.
+  constexpr int kWm = BM / 2, kWn = BN / 2, kQuads = kWn / 4;
+  f32x4* out = reinterpret_cast<f32x4*>(lds) + wave * kWm * kQuads;
 #pragma unroll
-  for (int i = 0; i < kTm; ++i) {
-    const int m = m0 + wm * (BM / 2) + i * 16 + (lane & 15);
-    if (m < g.M) {
+  for (int i = 0; i < kTm; ++i)
 #pragma unroll
-      for (int j = 0; j < kTn; ++j) {
-        const int n = n0 + wn * (BN / 2) + j * 16 + (lane >> 4) * 4;
-        if (n < N) epilogue<T>(g, group, m, n, acc[j][i]);
-      }
+    for (int j = 0; j < kTn; ++j) {
+      const int m = i * 16 + (lane & 15), quad = j * 4 + (lane >> 4);
+      out[m * kQuads + (quad ^ (m & (kQuads - 1)))] = acc[j][i];
     }
+#pragma unroll 1
+  for (int id = lane; id < kWm * kQuads; id += 64) {
+    const int r = id / kQuads, quad = id % kQuads, m = m0 + wm * kWm + r, n = n0 + wn * kWn + quad * 4;
+    if (m < g.M && n < N) epilogue<T>(g, group, m, n, out[r * kQuads + (quad ^ (r & (kQuads - 1)))]);
   }
 }
 

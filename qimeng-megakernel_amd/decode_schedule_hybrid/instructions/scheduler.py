@@ -21,7 +21,7 @@ MI355X_QUEUES = 256
 MAX_ROWS = 512             # rows of one instruction (pairs count as two)
 MIN_ROWS = 4
 KEYS_PER_PART = 64
-MAX_PARTS = 16
+MAX_PARTS = 32
 BARRIER_ROWS, BARRIER_SLOTS = 54, 48
 
 
