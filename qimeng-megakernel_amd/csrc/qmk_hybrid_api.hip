@@ -387,11 +387,11 @@ int prefill(const QmkHybridArgs* a) {
       d.f0 = b.fb; d.ldo = N;
       launch_gemm<T, u16, T>(d, st);
       const size_t step = static_cast<size_t>(P) * N;
-      const dim3 grid(n / 16, l.heads);
+      const dim3 grid(n / kWkvColumns, l.heads), lanes(kWkvThreads);
       const float *r = b.fa, *k = b.fa + step, *v = b.fa + 2 * step;
-      if (n <= 64) hipLaunchKernelGGL(wkv_scan<4>, grid, dim3(256), 0, st, r, k, v, b.fb, l, a->slot, M, b.raw);
-      else if (n <= 128) hipLaunchKernelGGL(wkv_scan<8>, grid, dim3(256), 0, st, r, k, v, b.fb, l, a->slot, M, b.raw);
-      else hipLaunchKernelGGL(wkv_scan<16>, grid, dim3(256), 0, st, r, k, v, b.fb, l, a->slot, M, b.raw);
+      if (n <= 64) hipLaunchKernelGGL((wkv_scan<4, 32>), grid, lanes, 0, st, r, k, v, b.fb, l, a->slot, M, b.raw);
+      else if (n <= 128) hipLaunchKernelGGL((wkv_scan<8, 16>), grid, lanes, 0, st, r, k, v, b.fb, l, a->slot, M, b.raw);
+      else hipLaunchKernelGGL((wkv_scan<16, 8>), grid, lanes, 0, st, r, k, v, b.fb, l, a->slot, M, b.raw);
       hipLaunchKernelGGL(wkv_out<T>, dim3((M * l.heads + 3) / 4), block, 0, st, b.raw, b.p0, l, M, a->eps, b.mix);
     }
     residual(l.o_w, W, l, false);

@@ -30,6 +30,7 @@ enum : int {
 constexpr int kMaxStreams = QMK_HYBRID_MAX_STREAMS;
 constexpr int kMaxTaps = QMK_HYBRID_MAX_TAPS;
 constexpr int kMaxRows = 512;                 // rows of one instruction
+constexpr int kMaxOutRows = kThreads / kMaxStreams;   // ... of OP_OUT_PROJECT: a thread per row and stream
 constexpr int kChunk = kWaveSize * 8;         // columns one wave covers with one 16-byte load per lane
 constexpr int kMaxK = 24576;                  // longest activation vector
 constexpr int kAttendFloats = 33792;          // LDS of the attention op: query, key tile, scores
@@ -37,10 +38,6 @@ constexpr int kMaxRank = 512;
 constexpr int kMaxHeadDim = 256;              // wkv
 constexpr int kMaxParts = 64;
 constexpr int kDepth = 8;                     // weight rows a wave keeps in flight and reduces together
-#ifndef QMK_EARLY
-#define QMK_EARLY 4
-#endif
-constexpr int kEarly = QMK_EARLY;
 constexpr int kAhead = 2;                     // quads of a vector a thread holds in registers (4096 elements a workgroup)
 constexpr int kStageGroupRows = 54;           // the counter layout of one group of four stages (qmk_device.h)
 constexpr int kStageGroupSlots = 48;
@@ -85,7 +82,6 @@ struct Smem {
     float attend[kAttendFloats];
   };
   float aux[3072];
-  float hc[kMaxStreams * (kMaxStreams + 3)];   // OP_OUT_PROJECT: output weights, mixes, the next sublayer's input weights
   float scratch[kWaves];
   int32_t inst[kInstWords];
   int32_t next_layer;
@@ -196,34 +192,28 @@ struct RowStream {
   }
   __device__ __forceinline__ void start(const u16* w, int rows, int columns) {
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / kWaveSize);
-    per = 1;
-    lanes = kWaveSize;
-    if ((columns == 128 && rows % 4 == 0) || (columns == 256 && rows % 2 == 0)) {
-      per = kChunk / columns;
-      lanes = kWaveSize / per;
-    }
+    int narrow = 0;                                          // log2 of the rows side by side
+    if (columns == 128 && rows % 4 == 0) narrow = 2;
+    if (columns == 256 && rows % 2 == 0) narrow = 1;
+    per = 1 << narrow;
+    lanes = kWaveSize >> narrow;
     ld = columns;
-    total = columns * per;
+    total = columns << narrow;
     pitch = total;
-    rows /= per;
-    const int chunks = (total + kChunk - 1) / kChunk;
-    const int share = chunks >= 4 ? (chunks == 4 ? 2 : 1) : (chunks == 1 ? 8 : chunks == 2 ? 4 : 2);   // waves per chunk
-    chunk = share == 1 ? wave : wave / share;
-    const int part = share == 1 ? 0 : wave - chunk * share;
-    first = rows * part / share;
-    n = rows * (part + 1) / share - first;
-    waves = chunk < chunks ? (chunks - chunk + kWaves - 1) / kWaves : 0;      // chunks of this wave: chunk, chunk + 8, ...
+    rows >>= narrow;
+    const unsigned chunks = static_cast<unsigned>(total + kChunk - 1) / kChunk;
+    const int share = chunks > 4 ? 0 : chunks > 2 ? 1 : chunks == 2 ? 2 : 3;     // log2 of the waves per chunk
+    chunk = wave >> share;
+    const int part = wave & ((1 << share) - 1);
+    first = (rows * part) >> share;
+    n = ((rows * (part + 1)) >> share) - first;
+    waves = chunk < static_cast<int>(chunks) ? (chunks - chunk + kWaves - 1) / kWaves : 0;      // chunks of this wave: chunk, chunk + 8, ...
     if (waves == 0) n = 0;
     at = w + first * pitch;
-    load_rows<0, kEarly>();
-  }
-  // Rows [from, to) of the first group
-  template <int from, int to>
-  __device__ __forceinline__ void load_rows() {
-    const u16* rows = at + column(chunk);
+    const u16* top = at + column(chunk);
 #pragma unroll
-    for (int j = from; j < to; ++j)
-      if (j < n) r[j] = __builtin_nontemporal_load(reinterpret_cast<const v4u*>(rows + j * pitch));
+    for (int j = 0; j < kDepth; ++j)
+      if (j < n) r[j] = __builtin_nontemporal_load(reinterpret_cast<const v4u*>(top + j * pitch));
   }
   // part[wave][row] += sums; part must be zero, one barrier behind it.
   __device__ __forceinline__ void run(Smem& s) {
@@ -443,6 +433,7 @@ __device__ __forceinline__ bool rows_of(const DecodeParams& p, LayerRef& l, cons
       return l.type == QMK_MIXER_WKV && o.sub >= 0 && o.sub < l.heads && l.head_dim <= kMaxHeadDim &&
              set(l.mid_w, static_cast<long long>(o.sub) * l.head_dim, l.head_dim, l.rank);
     case OP_OUT_PROJECT:
+      if (o.count > kMaxOutRows) return false;
       if (o.sub == 1) return l.has_mlp && o.start + o.count <= D && set(l.down_w, o.start, o.count, l.ff);
       return o.start + o.count <= D && set(l.o_w, o.start, o.count, l.mix_width);
     case OP_UP_GATE: return l.has_mlp && o.start + o.count <= l.ff && set(l.mlp_w, 2LL * o.start, 2 * o.count, D);
@@ -473,7 +464,8 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
   float* shift_new = l.shift + (static_cast<size_t>(p.slot) * 2 + 1 - p.flip) * shift_copy;
   const float* mu = l.vec2 + static_cast<size_t>(o.sub) * D;
   float4 w0[kAhead], w1[kAhead], w2[kAhead];
-  float a[kMaxStreams] = {};
+  float a[kMaxStreams] = {}, b[kMaxStreams] = {};
+  float out_weight = 0.f, next_weight = 0.f;
   float* state = nullptr;
   if (normed) {
     load_ahead(w0, norm, D);
@@ -517,26 +509,27 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
       w0[0] = make_float4(l.mid_b[at], l.vec1[at], l.vec0[at], 0.f);
     }
   } else if (op == OP_OUT_PROJECT) {
-    if (tid < S * (S + 2)) {
+    // Eight lanes per row, one per stream: all streams of the row, the stream's column of the mix, its output weight and
+    // its weight in the next sublayer's input.  Only this instruction touches its rows of the streams in this stage, and
+    // their last writer arrived stages ago.
+    const int r = o.start + (tid >> 3), q = tid & 7;
+    if ((tid >> 3) < m.rows && q < S) {
       const bool down = o.sub == 1;
-      s.hc[tid] = tid < S * (S + 1) ? l.hc[(down ? S * (S + 2) : 0) + S + tid] : (down ? l.next2 : l.next1)[tid - S * (S + 1)];
-    }
-    // Only this instruction touches its rows of the streams in this stage, and their last writer arrived stages ago.
-    if (mine) {
-      if (first) {
-        const float e = bf2f(p.embed[static_cast<size_t>(token_of(p)) * D + row]);
+      const float* hc = l.hc + (down ? S * (S + 2) : 0) + S;
+      const float e = first ? bf2f(p.embed[static_cast<size_t>(token_of(p)) * D + r]) : 0.f;
 #pragma unroll
-        for (int t = 0; t < kMaxStreams; ++t) a[t] = e;
-      } else {
-#pragma unroll
-        for (int t = 0; t < kMaxStreams; ++t)
-          if (t < S) a[t] = ld_shared_f32(p.x + static_cast<size_t>(t) * D + row);
+      for (int f = 0; f < kMaxStreams; ++f) {
+        if (f < S) {
+          a[f] = first ? e : ld_shared_f32(p.x + static_cast<size_t>(f) * D + r);
+          b[f] = hc[S + f * S + q];
+        }
       }
+      out_weight = hc[q];
+      next_weight = (down ? l.next2 : l.next1)[q];
     }
   }
   stamp(p, s, 0);
   if (!wait_stage(p, s, o)) return false;
-  g.load_rows<kEarly, kDepth>();
 
   // The activation vector.
   if (normed) {
@@ -570,17 +563,17 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
     static_assert(kMaxRank <= kThreads && kMaxParts <= kWaveSize, "one thread per latent element, one lane per part");
     const bool in = tid < l.rank;
     float v[kBatch];
-    auto request = [&](int base) {
+    const float* column = from + min(tid, l.rank - 1);
+    auto request = [&](int base) {   // no branches: sixteen requests leave back to back
 #pragma unroll
-      for (int j = 0; j < kBatch; ++j)
-        if (base + j < parts && in) v[j] = ld_shared_f32(from + (base + j) * pitch + tid);
+      for (int j = 0; j < kBatch; ++j) v[j] = ld_shared_f32(column + min(base + j, parts - 1) * pitch);
     };
     request(0);
     __syncthreads();
     if (tid < kWaveSize) {   // weights of the parts
       const float mx = tid < parts ? s.aux[tid] : -INFINITY, top = wave_max(mx);
       const float w = exp2_fast(mx - top), sum = wave_sum(tid < parts ? w * s.aux[kMaxParts + tid] : 0.f);
-      if (tid < parts) s.aux[tid] = w / sum;
+      s.aux[tid] = tid < parts ? w / sum : 0.f;
     }
     __syncthreads();
     float acc = 0.f;
@@ -588,8 +581,7 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
     for (int base = 0; base < parts; base += kBatch) {
       if (base != 0) request(base);
 #pragma unroll
-      for (int j = 0; j < kBatch; ++j)
-        if (base + j < parts) acc = fmaf(s.aux[base + j], v[j], acc);
+      for (int j = 0; j < kBatch; ++j) acc = fmaf(s.aux[base + j], v[j], acc);
     }
     if (in) s.xs[xs_at(tid)] = acc;
   } else {
@@ -620,21 +612,17 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
   stamp(p, s, 2);
 
   // What happens to the rows' sums; a pair of rows is a pair of lanes.
-  float t = mine ? row_total(s, tid) : 0.f;
+  float t = mine && op != OP_OUT_PROJECT ? row_total(s, tid) : 0.f;
   static_assert(kMaxRows <= kThreads && kMaxStreams == 8, "one row per thread, eight values ahead");
   if (op == OP_OUT_PROJECT) {
-    if (mine) {
-      float u = 0.f;
-#pragma unroll 1
-      for (int q = 0; q < S; ++q) {
-        float now = s.hc[q] * t;
+    const int r = tid >> 3, q = tid & 7;
+    if (r < m.rows) {      // whole groups of eight lanes
+      float now = out_weight * row_total(s, r);
 #pragma unroll
-        for (int f = 0; f < kMaxStreams; ++f)
-          if (f < S) now = fmaf(s.hc[S + f * S + q], a[f], now);
-        st_shared_f32(p.x + static_cast<size_t>(q) * D + row, now);
-        u = fmaf(s.hc[S * (S + 1) + q], now, u);
-      }
-      st_shared_f32(p.u + row, u);
+      for (int f = 0; f < kMaxStreams; ++f) now = fmaf(b[f], a[f], now);
+      const float u = group8_sum(next_weight * now);
+      if (q == 0) st_shared_f32(p.u + o.start + r, u);
+      if (q < S) st_shared_f32(p.x + static_cast<size_t>(q) * D + o.start + r, now);
     }
   } else if (op == OP_UP_GATE) {
     const float up = dpp_f32<kDppQuadXor1>(0.f, t);
@@ -812,14 +800,16 @@ __host__ __device__ constexpr int attend_floats(int row_elements, int element_by
 }
 
 // Part `start` of `count` of the visible keys, heads [16 sub, 16 sub + 16).  Scores: matrix tiles of 16 keys x 16 heads,
-// the row's columns split over the waves of a tile; then the weights and the running sums of weight x latent.
+// the row's columns split over the waves of a tile; then the weights and the running sums of weight x latent, of which an
+// instruction keeps columns [128 extra, 128 extra + 128), sixteen a wave.
 template <class T>
 __device__ __forceinline__ bool op_latent_attend(const DecodeParams& p, Smem& s, const Op& o) {
   constexpr int kKeys = attend_keys(sizeof(T)), kTiles = kKeys / 16, kSlices = kWaves / kTiles, kPer = kKeys * 16 / kThreads, kSp = kKeys + 8;
   constexpr int kUnit = 16 / sizeof(T);
   LayerRef& l = layer_of(p, o.layer);
   const int heads16 = (l.heads + 15) & ~15;
-  if (l.type != QMK_MIXER_LATENT || o.sub < 0 || o.sub * 16 >= l.heads || o.start < 0 || o.count <= 0 || o.count > p.max_splits || o.start >= o.count)
+  if (l.type != QMK_MIXER_LATENT || o.sub < 0 || o.sub * 16 >= l.heads || o.start < 0 || o.count <= 0 || o.count > p.max_splits || o.start >= o.count ||
+      o.extra < 0 || o.extra * 16 * kWaves >= l.rank)
     return bad_operand(p, o, o.start);
   const int tid = threadIdx.x, lane = tid & (kWaveSize - 1), wave = __builtin_amdgcn_readfirstlane(tid / kWaveSize);
   const int width = l.rank + l.rot_dim, width32 = (width + 31) & ~31, stride = width32 + 8;
@@ -890,8 +880,9 @@ __device__ __forceinline__ bool op_latent_attend(const DecodeParams& p, Smem& s,
   stamp(p, s, 1);
   const int head = tid & 15, key0 = tid >> 4;      // this thread's scores: keys key0, key0 + 32, ...
   float m = -INFINITY, lsum = 0.f;
-  f32x4 acc[kMaxRank / 16 / kWaves] = {};
-  const int tiles = l.rank / 16;
+  f32x4 acc = {};
+  const int column0 = (o.extra * kWaves + wave) * 16;      // this wave's sixteen columns of the latent
+  const bool columns = column0 < l.rank;
 #pragma unroll 1
   for (int base = lo; base < hi; base += kKeys) {
     if (base != lo) {
@@ -921,12 +912,17 @@ __device__ __forceinline__ bool op_latent_attend(const DecodeParams& p, Smem& s,
         for (int q = 0; q < kSlices; ++q) t += sred[(q * kKeys + key) * 16 + head];
         score[j] = t * (l.scale * kLog2e);
       }
-      ss[key * 16 + head] = score[j];
     }
+    float top = score[0];
+#pragma unroll
+    for (int j = 1; j < kPer; ++j) top = fmaxf(top, score[j]);
+    top = fmaxf(top, __shfl_xor(top, 16));
+    top = fmaxf(top, __shfl_xor(top, 32));
+    if (lane < 16) ss[wave * 16 + head] = top;
     __syncthreads();
-    float top = m;
-#pragma unroll 16
-    for (int k = 0; k < kKeys; ++k) top = fmaxf(top, ss[k * 16 + head]);
+    top = m;
+#pragma unroll
+    for (int k = 0; k < kWaves; ++k) top = fmaxf(top, ss[k * 16 + head]);
     const float shrink = exp2_fast(m - top);
     lsum *= shrink;
 #pragma unroll
@@ -938,21 +934,14 @@ __device__ __forceinline__ bool op_latent_attend(const DecodeParams& p, Smem& s,
     m = top;
     if (key0 == 0) sa[head] = shrink;
     __syncthreads();
-    {
-      const float a = sa[lane & 15];
+    if (columns) {
+      acc *= sa[lane & 15];
 #pragma unroll
-      for (int q = 0; q < kMaxRank / 16 / kWaves; ++q) {
-        const int t = q * kWaves + wave;
-        if (t < tiles) {
-          acc[q] *= a;
+      for (int kk = 0; kk < kKeys / 32; ++kk) {
+        Frag<T> cf;
 #pragma unroll
-          for (int kk = 0; kk < kKeys / 32; ++kk) {
-            Frag<T> cf;
-#pragma unroll
-            for (int j = 0; j < 8; ++j) cf.set(j, sc[(kk * 32 + (lane >> 4) * 8 + j) * stride + t * 16 + (lane & 15)]);
-            acc[q] = mma(cf, load_frag(sp + (lane & 15) * kSp + kk * 32 + (lane >> 4) * 8), acc[q]);
-          }
-        }
+        for (int j = 0; j < 8; ++j) cf.set(j, sc[(kk * 32 + (lane >> 4) * 8 + j) * stride + column0 + (lane & 15)]);
+        acc = mma(cf, load_frag(sp + (lane & 15) * kSp + kk * 32 + (lane >> 4) * 8), acc);
       }
     }
     __syncthreads();
@@ -964,24 +953,19 @@ __device__ __forceinline__ bool op_latent_attend(const DecodeParams& p, Smem& s,
   if (lane < 16) ss[wave * 16 + head] = lsum;
   __syncthreads();
   float* ml = p.ml + (static_cast<size_t>(o.start) * heads16 + o.sub * 16) * 2;
-  if (key0 == 0) {
+  if (key0 == 0 && o.extra == 0) {
     float t = 0.f;
 #pragma unroll
     for (int k = 0; k < kWaves; ++k) t += ss[k * 16 + head];
     st_shared_f32(ml + head * 2, m);
     st_shared_f32(ml + head * 2 + 1, t);
   }
-  float* out = p.part + (static_cast<size_t>(o.start) * heads16 + o.sub * 16 + (lane & 15)) * l.rank;
+  if (columns) {
+    uint64_t* at = reinterpret_cast<uint64_t*>(p.part + (static_cast<size_t>(o.start) * heads16 + o.sub * 16 + (lane & 15)) * l.rank + column0 + (lane >> 4) * 4);
 #pragma unroll
-  for (int q = 0; q < kMaxRank / 16 / kWaves; ++q) {
-    const int t = q * kWaves + wave;
-    if (t < tiles) {
-      uint64_t* at = reinterpret_cast<uint64_t*>(out + t * 16 + (lane >> 4) * 4);
-#pragma unroll
-      for (int i = 0; i < 2; ++i)
-        __hip_atomic_store(at + i, (static_cast<uint64_t>(__float_as_uint(acc[q][2 * i + 1])) << 32) | __float_as_uint(acc[q][2 * i]), __ATOMIC_RELAXED,
-                           __HIP_MEMORY_SCOPE_AGENT);
-    }
+    for (int i = 0; i < 2; ++i)
+      __hip_atomic_store(at + i, (static_cast<uint64_t>(__float_as_uint(acc[2 * i + 1])) << 32) | __float_as_uint(acc[2 * i]), __ATOMIC_RELAXED,
+                         __HIP_MEMORY_SCOPE_AGENT);
   }
   stamp(p, s, 3);
   arrive_stage(p, o);

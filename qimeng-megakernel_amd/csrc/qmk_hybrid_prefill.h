@@ -531,54 +531,89 @@ __global__ __launch_bounds__(kPfThreads) void window_attention(const T* q, const
     if (t < vt) store4(out + at + t * 16 + g * 4, acc[t] * inv * read4(gate + at + t * 16 + g * 4));
 }
 
-// The wkv recurrence: one head and sixteen value columns a workgroup; sixteen lanes share a column's key rows.
-constexpr int kWkvTokens = 16, kWkvKeys = kMaxHeadDim / 16;
-template <int KPL>   // key rows per lane (head size up to 16 KPL)
-__global__ __launch_bounds__(256) void wkv_scan(const float* r, const float* k, const float* v, const float* w, QmkHybridLayer l, int slot, int M, float* out) {
-  __shared__ float sr[kWkvTokens][16 * KPL], sk[kWkvTokens][16 * KPL], sw[kWkvTokens][16 * KPL], sv[kWkvTokens][16];
-  const int n = l.head_dim, N = l.heads * n, head = blockIdx.y, v0 = blockIdx.x * 16;
+// The wkv recurrence: one head and eight value columns a workgroup; sixteen lanes share a column, KPL neighbouring key
+// rows each, in registers.  TB tokens at a time: the next block's r, k, w, v are in flight while this one runs, a block's
+// outputs leave together.  Places behind the last token or key row hold r = k = 0, w = 1, which changes nothing.
+constexpr int kWkvColumns = 8, kWkvThreads = 16 * kWkvColumns;
+template <int KPL, int TB>
+__global__ __launch_bounds__(kWkvThreads) void wkv_scan(const float* r, const float* k, const float* v, const float* w, QmkHybridLayer l, int slot, int M, float* out) {
+  constexpr int kKeys = 16 * KPL, kQuads = TB * kKeys / 4 / kWkvThreads, kValueQuads = TB * kWkvColumns / 4;
+  static_assert(kQuads * kWkvThreads * 4 == TB * kKeys && kValueQuads <= kWkvThreads, "every thread stages the same number of quads");
+  __shared__ __align__(16) float sr[2][TB][kKeys], sk[2][TB][kKeys], sw[2][TB][kKeys], sv[2][TB][kWkvColumns], so[2][TB][kWkvColumns];
+  const int n = l.head_dim, N = l.heads * n, head = blockIdx.y, v0 = blockIdx.x * kWkvColumns;
   const int tid = threadIdx.x, part = tid & 15, e = tid >> 4;
-  float* st = l.state + (static_cast<size_t>(slot) * l.heads + head) * n * n;
+  float* st = l.state + (static_cast<size_t>(slot) * l.heads + head) * n * n + v0 + e;
   float s[KPL], u[KPL];
 #pragma unroll
   for (int i = 0; i < KPL; ++i) {
-    const int row = i * 16 + part;
-    s[i] = row < n ? st[row * n + v0 + e] : 0.f;
+    const int row = part * KPL + i;
+    s[i] = row < n ? st[row * n] : 0.f;
     u[i] = row < n ? l.vec1[head * n + row] : 0.f;
   }
-  for (int base = 0; base < M; base += kWkvTokens) {
-    const int count = min(kWkvTokens, M - base);
-    __syncthreads();
-    for (int i = tid; i < count * 16 * KPL; i += 256) {
-      const int t = i / (16 * KPL), c = i % (16 * KPL);
-      const size_t at = static_cast<size_t>(base + t) * N + head * n + c;
-      sr[t][c] = c < n ? r[at] : 0.f;
-      sk[t][c] = c < n ? k[at] : 0.f;
-      sw[t][c] = c < n ? w[at] : 0.f;
+  f32x4 fr[kQuads], fk[kQuads], fw[kQuads], fv = {};
+  auto fetch = [&](int base) {
+#pragma unroll
+    for (int q = 0; q < kQuads; ++q) {
+      const int id = tid + q * kWkvThreads, t = base + id / (kKeys / 4), c = id % (kKeys / 4) * 4;
+      const size_t at = static_cast<size_t>(t) * N + head * n + c;
+      const bool real = t < M && c < n;
+      fr[q] = real ? *reinterpret_cast<const f32x4*>(r + at) : f32x4{0.f, 0.f, 0.f, 0.f};
+      fk[q] = real ? *reinterpret_cast<const f32x4*>(k + at) : f32x4{0.f, 0.f, 0.f, 0.f};
+      fw[q] = real ? *reinterpret_cast<const f32x4*>(w + at) : f32x4{1.f, 1.f, 1.f, 1.f};
     }
-    if (e < count) sv[e][part] = v[static_cast<size_t>(base + e) * N + head * n + v0 + part];
-    __syncthreads();
-    for (int t = 0; t < count; ++t) {
-      const float vt = sv[t][e];
+    if (tid < kValueQuads) {
+      const int t = base + tid / (kWkvColumns / 4);
+      fv = t < M ? *reinterpret_cast<const f32x4*>(v + static_cast<size_t>(t) * N + head * n + v0 + tid % (kWkvColumns / 4) * 4) : f32x4{0.f, 0.f, 0.f, 0.f};
+    }
+  };
+  auto stash = [&](int buf) {
+#pragma unroll
+    for (int q = 0; q < kQuads; ++q) {
+      const int id = tid + q * kWkvThreads, t = id / (kKeys / 4), c = id % (kKeys / 4) * 4;
+      *reinterpret_cast<f32x4*>(&sr[buf][t][c]) = fr[q];
+      *reinterpret_cast<f32x4*>(&sk[buf][t][c]) = fk[q];
+      *reinterpret_cast<f32x4*>(&sw[buf][t][c]) = fw[q];
+    }
+    if (tid < kValueQuads) *reinterpret_cast<f32x4*>(&sv[buf][tid / (kWkvColumns / 4)][tid % (kWkvColumns / 4) * 4]) = fv;
+  };
+  fetch(0);
+  stash(0);
+  __syncthreads();
+  int buf = 0;
+  for (int base = 0; base < M; base += TB, buf ^= 1) {
+    if (base + TB < M) fetch(base + TB);
+#pragma unroll 4
+    for (int t = 0; t < TB; ++t) {
+      const float vt = sv[buf][t][e];
       float o = 0.f;
 #pragma unroll
-      for (int i = 0; i < KPL; ++i) {
-        const int row = i * 16 + part;
-        const float kv = sk[t][row] * vt;
-        o = fmaf(sr[t][row], fmaf(u[i], kv, s[i]), o);
-        s[i] = fmaf(sw[t][row], s[i], kv);
+      for (int i = 0; i < KPL; i += 4) {
+        const f32x4 r4 = *reinterpret_cast<const f32x4*>(&sr[buf][t][part * KPL + i]), k4 = *reinterpret_cast<const f32x4*>(&sk[buf][t][part * KPL + i]),
+                    w4 = *reinterpret_cast<const f32x4*>(&sw[buf][t][part * KPL + i]);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const float kv = k4[j] * vt;
+          o = fmaf(r4[j], fmaf(u[i + j], kv, s[i + j]), o);
+          s[i + j] = fmaf(w4[j], s[i + j], kv);
+        }
       }
       o += dpp_f32<kDppQuadXor1>(0.f, o);
       o += dpp_f32<kDppQuadXor2>(0.f, o);
       o += dpp_f32<kDppHalfMirror>(0.f, o);
       o += dpp_f32<0x140>(0.f, o);            // row_mirror: lane i <-> 15-i of its sixteen
-      if (part == 0) out[static_cast<size_t>(base + t) * N + head * n + v0 + e] = o;
+      if (part == 0) so[buf][t][e] = o;
+    }
+    if (base + TB < M) stash(buf ^ 1);
+    __syncthreads();
+    for (int id = tid; id < TB * kWkvColumns; id += kWkvThreads) {
+      const int t = id / kWkvColumns, c = id % kWkvColumns;
+      if (base + t < M) out[static_cast<size_t>(base + t) * N + head * n + v0 + c] = so[buf][t][c];
     }
   }
 #pragma unroll
   for (int i = 0; i < KPL; ++i) {
-    const int row = i * 16 + part;
-    if (row < n) st[row * n + v0 + e] = s[i];
+    const int row = part * KPL + i;
+    if (row < n) st[row * n] = s[i];
   }
 }
 

@@ -54,6 +54,7 @@ class LatentAbsorb(StageInstruction):
 
 @dataclass
 class LatentAttendSplitKV(StageInstruction):
+    """``extra``: which 128 columns of the latent."""
     OPCODE: ClassVar[int] = 4
 
 

@@ -19,9 +19,11 @@ from . import instruction_defs as D
 
 MI355X_QUEUES = 256
 MAX_ROWS = 512             # rows of one instruction (pairs count as two)
+MAX_OUT_ROWS = 64          # ... of an output projection: a thread per row and stream
 MIN_ROWS = 4
 KEYS_PER_PART = 64
 MAX_PARTS = 32
+ATTEND_COLUMNS = 128       # latent columns one attention instruction sums up
 BARRIER_ROWS, BARRIER_SLOTS = 54, 48
 
 
@@ -70,13 +72,14 @@ class HybridScheduler:
             stages.append([D.LatentAbsorb(i, h, a, n) for h, a, n in cut([(h, l.rank_s) for h in range(l.heads)], q)])
             stages[-1][0].extra = 1
             parts = self.parts(i)
-            stages.append([D.LatentAttendSplitKV(i, g, part, parts) for g in range(_ceil_div(l.heads, 16)) for part in range(parts)])
+            stages.append([D.LatentAttendSplitKV(i, g, part, parts, extra=c) for g in range(_ceil_div(l.heads, 16)) for part in range(parts)
+                           for c in range(_ceil_div(l.rank_s, ATTEND_COLUMNS))])
             stages.append([D.LatentValue(i, h, a, n, extra=parts) for h, a, n in cut([(h, l.v_s) for h in range(l.heads)], q)])
         D_s = self.shape.width_s
-        stages.append([D.OutProject_Streams(i, 0, a, n) for _, a, n in cut([(0, D_s)], q)])
+        stages.append([D.OutProject_Streams(i, 0, a, n) for _, a, n in cut([(0, D_s)], q, most=MAX_OUT_ROWS)])
         if l.ff:
             stages.append([D.RMS_UpGate_Gelu(i, 0, a, n) for _, a, n in cut([(0, l.ff_s)], q, most=MAX_ROWS // 2)])
-            stages.append([D.OutProject_Streams(i, 1, a, n) for _, a, n in cut([(0, D_s)], q)])
+            stages.append([D.OutProject_Streams(i, 1, a, n) for _, a, n in cut([(0, D_s)], q, most=MAX_OUT_ROWS)])
         return stages
 
     def stages(self) -> list[list[D.StageInstruction]]:
