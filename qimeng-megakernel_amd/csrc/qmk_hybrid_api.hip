@@ -313,11 +313,18 @@ size_t prefill_buffers(const QmkHybridArgs* a, void* base, PrefillBuffers<T>* b)
 template <class TA, class TW, class T>
 void launch_gemm(const GemmArgs& g, hipStream_t st) {
   const int n = std::max(g.N, g.last_n);
-  auto tiles = [&](int bm, int bn) { return static_cast<long long>((g.M + bm - 1) / bm) * ((n + bn - 1) / bn) * g.groups; };
-  if (tiles(128, 128) >= 192)
-    hipLaunchKernelGGL((gemm<TA, TW, T, 128, 128>), dim3((n + 127) / 128, (g.M + 127) / 128, g.groups), dim3(kPfThreads), 0, st, g);
-  else
-    hipLaunchKernelGGL((gemm<TA, TW, T, 64, 64>), dim3((n + 63) / 64, (g.M + 63) / 64, g.groups), dim3(kPfThreads), 0, st, g);
+  auto grid = [&](int bm, int bn) { return dim3((n + bn - 1) / bn, (g.M + bm - 1) / bm, g.groups); };
+  const dim3 large = grid(128, 128), block(kPfThreads);
+  const bool fills = static_cast<long long>(large.x) * large.y * large.z >= 192;
+  if constexpr (sizeof(TA) == 2 && sizeof(TW) == 2) {
+    if (g.K % 64 == 0) {
+      if (fills) hipLaunchKernelGGL((gemm_direct<T, 128, 128, 2>), large, block, 0, st, g);
+      else hipLaunchKernelGGL((gemm_direct<T, 64, 64, 4>), grid(64, 64), block, 0, st, g);
+      return;
+    }
+  }
+  if (fills) hipLaunchKernelGGL((gemm<TA, TW, T, 128, 128>), large, block, 0, st, g);
+  else hipLaunchKernelGGL((gemm<TA, TW, T, 64, 64>), grid(64, 64), block, 0, st, g);
 }
 
 template <class T, int QT, int VT>

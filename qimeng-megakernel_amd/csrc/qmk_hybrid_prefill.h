@@ -174,6 +174,34 @@ __device__ __forceinline__ void epilogue(const GemmArgs& g, int group, int m, in
   }
 }
 
+// A workgroup's accumulators -> epilogue, through LDS (a wave's own part, quads of a row exchanged by its number): a lane's
+// accumulators are then read back in a loop, and the lanes of a row write neighbouring outputs of one token.
+template <class T, int BM, int BN, int kTn, int kTm>
+__device__ __forceinline__ void finish_tile(const GemmArgs& g, int group, int m0, int n0, int N, v4u* lds, const f32x4 (&acc)[kTn][kTm]) {
+  constexpr int kWm = BM / 2, kWn = BN / 2, kQuads = kWn / 4;
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, wm = wave & 1, wn = wave >> 1;
+  f32x4* out = reinterpret_cast<f32x4*>(lds) + wave * kWm * kQuads;
+#pragma unroll
+  for (int i = 0; i < kTm; ++i)
+#pragma unroll
+    for (int j = 0; j < kTn; ++j) {
+      const int m = i * 16 + (lane & 15), quad = j * 4 + (lane >> 4);
+      out[m * kQuads + (quad ^ (m & (kQuads - 1)))] = acc[j][i];
+    }
+#pragma unroll 1
+  for (int id = lane; id < kWm * kQuads; id += 64) {
+    const int r = id / kQuads, quad = id % kQuads, m = m0 + wm * kWm + r, n = n0 + wn * kWn + quad * 4;
+    if (m < g.M && n < N) epilogue<T>(g, group, m, n, out[r * kQuads + (quad ^ (r & (kQuads - 1)))]);
+  }
+}
+
+// Until at most `n` of this wave's vector-memory requests are outstanding and none of its LDS reads.
+template <int n>
+__device__ __forceinline__ void wait_outstanding() {
+  static_assert(n >= 0 && n < 64, "six bits");
+  asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)" ::"n"(n) : "memory");
+}
+
 // out[m][n] = sum_k a[m][k] w[n][k]: BN weight rows x BM tokens per workgroup, four waves as 2 x 2, 64 columns a step.
 // The weights are the matrix instruction's first operand, so a lane ends up with four consecutive outputs of one token.
 // LDS tiles hold 16-byte units, a row's units rotated by the row number (conflict-free fragment reads).
@@ -252,22 +280,79 @@ __global__ __launch_bounds__(kPfThreads) void gemm(const GemmArgs g) {
     if (s + 1 < steps) stash(buf ^ 1);
     __syncthreads();
   }
-  // Through LDS (a wave's own 64 x 64 part, quads of a row exchanged by its number): a lane's accumulators are then read
-  // back in a loop, and sixteen lanes write 64 neighbouring outputs of one token.
-  constexpr int kWm = BM / 2, kWn = BN / 2, kQuads = kWn / 4;
-  f32x4* out = reinterpret_cast<f32x4*>(lds) + wave * kWm * kQuads;
+  finish_tile<T, BM, BN>(g, group, m0, n0, N, lds, acc);
+}
+
+// The same for bf16 x bf16 with K a multiple of 64: tiles go from memory to LDS without passing through registers, STAGES
+// buffers deep, so that STAGES - 1 steps are in flight while one is multiplied.
+template <class T, int BM, int BN, int STAGES>
+__global__ __launch_bounds__(kPfThreads) void gemm_direct(const GemmArgs g) {
+  constexpr int kBK = 64, kRow = kBK / 8;                                   // a row: eight units of 16 bytes
+  constexpr int kLoads = (BM + BN) * kRow / kPfThreads, kStageUnits = (BM + BN) * kRow;
+  constexpr int kTm = BM / 2 / 16, kTn = BN / 2 / 16, kOutUnits = BM * BN / 4, kAhead = STAGES - 1;
+  __shared__ __align__(16) v4u lds[STAGES * kStageUnits > kOutUnits ? STAGES * kStageUnits : kOutUnits];
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), wm = wave & 1, wn = wave >> 1;
+  const int group = blockIdx.z;
+  const int N = group == g.groups - 1 ? g.last_n : g.N;
+  const int m0 = blockIdx.y * BM, n0 = blockIdx.x * BN;
+  if (n0 >= N) return;
+  const u16* a = static_cast<const u16*>(g.a) + group * g.a_step;
+  const u16* w = static_cast<const u16*>(g.w) + group * g.w_step;
+
+  // This thread's places in a stage: unit i * 256 + tid, tokens first.  A row's units are exchanged by its number, here on
+  // the memory side: the LDS side of such a load is one run of 64 units per wave.
+  const u16* from[kLoads];
 #pragma unroll
-  for (int i = 0; i < kTm; ++i)
-#pragma unroll
-    for (int j = 0; j < kTn; ++j) {
-      const int m = i * 16 + (lane & 15), quad = j * 4 + (lane >> 4);
-      out[m * kQuads + (quad ^ (m & (kQuads - 1)))] = acc[j][i];
-    }
-#pragma unroll 1
-  for (int id = lane; id < kWm * kQuads; id += 64) {
-    const int r = id / kQuads, quad = id % kQuads, m = m0 + wm * kWm + r, n = n0 + wn * kWn + quad * 4;
-    if (m < g.M && n < N) epilogue<T>(g, group, m, n, out[r * kQuads + (quad ^ (r & (kQuads - 1)))]);
+  for (int i = 0; i < kLoads; ++i) {
+    const int id = i * kPfThreads + tid, r = id / kRow, c = ((id % kRow) ^ (r & 7)) * 8;
+    from[i] = r < BM ? a + static_cast<size_t>(min(m0 + r, g.M - 1)) * g.lda + c : w + static_cast<size_t>(min(n0 + r - BM, N - 1)) * g.ldw + c;
   }
+  auto issue = [&](int buf) {
+#pragma unroll
+    for (int i = 0; i < kLoads; ++i) {
+      const auto* src = (const __attribute__((address_space(1))) uint32_t*)from[i];
+      auto* dst = (__attribute__((address_space(3))) uint32_t*)(lds + buf * kStageUnits + i * kPfThreads + wave * 64);
+      __builtin_amdgcn_global_load_lds(src, dst, 16, 0, 0);
+      from[i] += kBK;
+    }
+  };
+  f32x4 acc[kTn][kTm] = {};
+  const int steps = g.K / kBK;
+#pragma unroll
+  for (int s = 0; s < kAhead; ++s)
+    if (s < steps) issue(s);
+  int buf = 0;
+  for (int s = 0; s < steps; ++s) {
+    // Everything up to this step's stage has landed; the barrier makes that true of every wave's part, and says that the
+    // buffer filled next is no longer read.
+    if (s + kAhead - 1 < steps) wait_outstanding<(kAhead - 1) * kLoads>();
+    else wait_outstanding<0>();
+    __builtin_amdgcn_s_barrier();
+    asm volatile("" ::: "memory");
+    if (s + kAhead < steps) issue(buf == 0 ? STAGES - 1 : buf - 1);
+    const v4u* la = lds + buf * kStageUnits;
+    const v4u* lw = la + BM * kRow;
+#pragma unroll
+    for (int kk = 0; kk < 2; ++kk) {
+      const int q = kk * 4 + (lane >> 4);
+      Frag<u16> fa[kTm];
+#pragma unroll
+      for (int i = 0; i < kTm; ++i) {
+        const int r = wm * (BM / 2) + i * 16 + (lane & 15);
+        fa[i] = load_frag(reinterpret_cast<const u16*>(la + r * kRow + (q ^ (r & 7))));
+      }
+#pragma unroll
+      for (int j = 0; j < kTn; ++j) {
+        const int r = wn * (BN / 2) + j * 16 + (lane & 15);
+        const Frag<u16> fw = load_frag(reinterpret_cast<const u16*>(lw + r * kRow + (q ^ (r & 7))));
+#pragma unroll
+        for (int i = 0; i < kTm; ++i) acc[j][i] = mma(fw, fa[i], acc[j][i]);
+      }
+    }
+    buf = buf + 1 == STAGES ? 0 : buf + 1;
+  }
+  __syncthreads();
+  finish_tile<T, BM, BN>(g, group, m0, n0, N, lds, acc);
 }
 
 __device__ __forceinline__ float pf_block_sum(float v, float* scratch) {
