@@ -539,30 +539,63 @@ __global__ __launch_bounds__(kPfThreads) void window_attention(const T* q, const
   const int lo = max(first, position + q0 + 1 - l.window);      // the first key any of the 64 queries sees
   const int hi = min(position + q0 + 64, position + M);          // behind the last one
   constexpr int kU = 16 / sizeof(T);
-  for (int base = first + ((lo - first) & ~(kKeys - 1)); base < hi; base += kKeys) {
-    const int ku = dq / kU;
-    for (int i = tid; i < kKeys * ku; i += kPfThreads) {
-      const int r = i / ku, c = (i - r * ku) * kU, row = base + r - first;
-      v4u v = {0u, 0u, 0u, 0u};
-      if (base + r < hi) {
-        if (c < l.head_dim) v = *reinterpret_cast<const v4u*>(k_nope + static_cast<size_t>(row) * l.heads * l.head_dim + head * l.head_dim + c);
-        else if (c < l.head_dim + l.rot_dim) v = *reinterpret_cast<const v4u*>(rows + static_cast<size_t>(row) * width + l.rank + c - l.head_dim);
-      }
-      *reinterpret_cast<v4u*>(&sk[r][c]) = v;
+  // Staging: each thread has fixed places in a tile of keys and of transposed values; the next tile is in flight while
+  // this one is used.
+  constexpr int kKLoads = kKeys * QT * 32 / kU / kPfThreads, kVLoads = VT * 16 * kKeys / kU / kPfThreads;
+  static_assert(kKLoads * kPfThreads * kU == kKeys * QT * 32 && kVLoads * kPfThreads * kU == VT * 16 * kKeys, "every thread stages the same number of units");
+  const int base0 = first + ((lo - first) & ~(kKeys - 1));
+  const T* k_at[kKLoads];
+  int k_step[kKLoads];
+  v4u rk[kKLoads], rv[kVLoads];
+#pragma unroll
+  for (int i = 0; i < kKLoads; ++i) {
+    const int id = i * kPfThreads + tid, r = id / (QT * 32 / kU), c = id % (QT * 32 / kU) * kU, row = base0 + r - first;
+    k_at[i] = nullptr;                 // columns behind the rotated part: zeros
+    k_step[i] = 0;
+    if (c < l.head_dim) {
+      k_at[i] = k_nope + static_cast<size_t>(row) * l.heads * l.head_dim + head * l.head_dim + c;
+      k_step[i] = kKeys * l.heads * l.head_dim;
+    } else if (c < l.head_dim + l.rot_dim) {
+      k_at[i] = rows + static_cast<size_t>(row) * width + l.rank + c - l.head_dim;
+      k_step[i] = kKeys * width;
     }
-    const int vu = kKeys / kU;
-    for (int i = tid; i < l.v_dim * vu; i += kPfThreads) {
-      const int r = i / vu, c = (i - r * vu) * kU;
-      v4u v = *reinterpret_cast<const v4u*>(v_t + static_cast<size_t>(head * l.v_dim + r) * keys_cap + base - first + c);
+  }
+  auto fetch = [&](int base) {
+#pragma unroll
+    for (int i = 0; i < kKLoads; ++i) {
+      const int r = (i * kPfThreads + tid) / (QT * 32 / kU);
+      rk[i] = v4u{0u, 0u, 0u, 0u};
+      if (k_at[i] != nullptr && base + r < hi) rk[i] = *reinterpret_cast<const v4u*>(k_at[i]);
+      k_at[i] = k_at[i] == nullptr ? nullptr : k_at[i] + k_step[i];
+    }
+#pragma unroll
+    for (int i = 0; i < kVLoads; ++i) {
+      const int id = i * kPfThreads + tid, r = id / (kKeys / kU), c = id % (kKeys / kU) * kU;
+      rv[i] = v4u{0u, 0u, 0u, 0u};
+      if (r < l.v_dim && base + c < hi) rv[i] = *reinterpret_cast<const v4u*>(v_t + static_cast<size_t>(head * l.v_dim + r) * keys_cap + base - first + c);
       if (base + c + kU > hi) {   // keys behind the last one: whatever the buffer holds there must not enter a sum
-        T* e = reinterpret_cast<T*>(&v);
+        T* e = reinterpret_cast<T*>(&rv[i]);
 #pragma unroll
         for (int j = 0; j < kU; ++j)
           if (base + c + j >= hi) e[j] = from_f32<T>(0.f);
       }
-      *reinterpret_cast<v4u*>(&sv[r][c]) = v;
+    }
+  };
+  fetch(base0);
+  const int first_pos = position + q0 + wave * 16;       // this wave's queries: first_pos .. first_pos + 15
+  for (int base = base0; base < hi; base += kKeys) {
+#pragma unroll
+    for (int i = 0; i < kKLoads; ++i) {
+      const int id = i * kPfThreads + tid;
+      *reinterpret_cast<v4u*>(&sk[id / (QT * 32 / kU)][id % (QT * 32 / kU) * kU]) = rk[i];
+    }
+#pragma unroll
+    for (int i = 0; i < kVLoads; ++i) {
+      const int id = i * kPfThreads + tid;
+      *reinterpret_cast<v4u*>(&sv[id / (kKeys / kU)][id % (kKeys / kU) * kU]) = rv[i];
     }
     __syncthreads();
+    if (base + kKeys < hi) fetch(base + kKeys);
     f32x4 d[2] = {};
 #pragma unroll
     for (int s = 0; s < QT; ++s)
@@ -573,11 +606,16 @@ __global__ __launch_bounds__(kPfThreads) void window_attention(const T* q, const
     float w[8];
     float best = top;
 #pragma unroll
-    for (int j = 0; j < 8; ++j) {
-      const int key = base + (j >> 2) * 16 + g * 4 + (j & 3), dist = pos - key;
-      w[j] = dist >= 0 && dist < l.window ? d[j >> 2][j & 3] * scale : -INFINITY;
-      best = fmaxf(best, w[j]);
+    for (int j = 0; j < 8; ++j) w[j] = d[j >> 2][j & 3] * scale;
+    if (base + kKeys - 1 > first_pos || first_pos + 15 - base >= l.window) {   // some query does not see some key
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        const int key = base + (j >> 2) * 16 + g * 4 + (j & 3), dist = pos - key;
+        if (dist < 0 || dist >= l.window) w[j] = -INFINITY;
+      }
     }
+#pragma unroll
+    for (int j = 0; j < 8; ++j) best = fmaxf(best, w[j]);
     best = fmaxf(best, __shfl_xor(best, 16));
     best = fmaxf(best, __shfl_xor(best, 32));
     const float ref = best == -INFINITY ? 0.f : best;      // no key of this query yet
@@ -667,26 +705,34 @@ __global__ __launch_bounds__(kWkvThreads) void wkv_scan(const float* r, const fl
   int buf = 0;
   for (int base = 0; base < M; base += TB, buf ^= 1) {
     if (base + TB < M) fetch(base + TB);
-#pragma unroll 4
-    for (int t = 0; t < TB; ++t) {
-      const float vt = sv[buf][t][e];
-      float o = 0.f;
+    // Four tokens at a time: their sums over the sixteen lanes are taken together (two steps that halve the values while
+    // they pair lanes, then plain sums), and lane p of sixteen ends up with token p % 4.
+    for (int t0 = 0; t0 < TB; t0 += 4) {
+      float o[4];
 #pragma unroll
-      for (int i = 0; i < KPL; i += 4) {
-        const f32x4 r4 = *reinterpret_cast<const f32x4*>(&sr[buf][t][part * KPL + i]), k4 = *reinterpret_cast<const f32x4*>(&sk[buf][t][part * KPL + i]),
-                    w4 = *reinterpret_cast<const f32x4*>(&sw[buf][t][part * KPL + i]);
+      for (int q = 0; q < 4; ++q) {
+        const int t = t0 + q;
+        const float vt = sv[buf][t][e];
+        o[q] = 0.f;
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          const float kv = k4[j] * vt;
-          o = fmaf(r4[j], fmaf(u[i + j], kv, s[i + j]), o);
-          s[i + j] = fmaf(w4[j], s[i + j], kv);
+        for (int i = 0; i < KPL; i += 4) {
+          const f32x4 r4 = *reinterpret_cast<const f32x4*>(&sr[buf][t][part * KPL + i]), k4 = *reinterpret_cast<const f32x4*>(&sk[buf][t][part * KPL + i]),
+                      w4 = *reinterpret_cast<const f32x4*>(&sw[buf][t][part * KPL + i]);
+#pragma unroll
+          for (int j = 0; j < 4; ++j) {
+            const float kv = k4[j] * vt;
+            o[q] = fmaf(r4[j], fmaf(u[i + j], kv, s[i + j]), o[q]);
+            s[i + j] = fmaf(w4[j], s[i + j], kv);
+          }
         }
       }
-      o += dpp_f32<kDppQuadXor1>(0.f, o);
-      o += dpp_f32<kDppQuadXor2>(0.f, o);
-      o += dpp_f32<kDppHalfMirror>(0.f, o);
-      o += dpp_f32<0x140>(0.f, o);            // row_mirror: lane i <-> 15-i of its sixteen
-      if (part == 0) so[buf][t][e] = o;
+      const bool b0 = part & 1, b1 = part & 2;
+      const float lo = (b0 ? o[1] : o[0]) + dpp_f32<kDppQuadXor1>(0.f, b0 ? o[0] : o[1]);
+      const float hi = (b0 ? o[3] : o[2]) + dpp_f32<kDppQuadXor1>(0.f, b0 ? o[2] : o[3]);
+      float sum = (b1 ? hi : lo) + dpp_f32<kDppQuadXor2>(0.f, b1 ? lo : hi);
+      sum += dpp_f32<0x124>(0.f, sum);        // row_ror:4
+      sum += dpp_f32<0x128>(0.f, sum);        // row_ror:8
+      if (part < 4) so[buf][t0 + part][e] = sum;
     }
     if (base + TB < M) stash(buf ^ 1);
     __syncthreads();
