@@ -109,8 +109,8 @@ class HybridMegaKernel:
         self._source: tuple[torch.Tensor, int] | None = None
 
     def _bind(self, g: Globals) -> None:
-        if g.instructions is None:
-            _scheduler.build(g)
+        if g.instructions is None:   # a step needs all its workgroups on the chip at once
+            _scheduler.build(g, max(1, min(_scheduler.MI355X_QUEUES, int(self._lib.qmk_hybrid_max_queues()))))
         key = (id(g), g.instructions.data_ptr(), g.barriers.data_ptr())
         if key == self._key:
             return

@@ -370,11 +370,12 @@ def random_hybrid_weights(shape: HybridShape, seed: int, device: torch.device | 
 
 
 def build_synthetic_hybrid_globals(shape: HybridShape, *, seed: int = 0, max_positions: int = 1032, slots: int = 1, portion_rows: int = 2048,
-                                   dtype: torch.dtype = torch.bfloat16, device: torch.device | str = "cuda") -> Any:
-    """Convenience: weights of ``seed`` drawn on ``device``, states and buffers of the hybrid route."""
+                                   dtype: torch.dtype = torch.bfloat16, device: torch.device | str = "cuda", draw_on: torch.device | str | None = None) -> Any:
+    """Convenience: weights of ``seed`` (drawn on ``device`` unless ``draw_on`` says otherwise), states and buffers of the
+    hybrid route."""
     from .decode_schedule_hybrid import HybridConfig, weights
     from .decode_schedule_hybrid.globs import build_globals as build_hybrid
 
     HybridConfig.set_shape(shape)
-    packed = weights.pack(shape, random_hybrid_weights(shape, seed, device), device)
+    packed = weights.pack(shape, random_hybrid_weights(shape, seed, draw_on or device), device)
     return build_hybrid(shape, packed, dtype=dtype, slots=slots, max_positions=max_positions, portion_rows=portion_rows)

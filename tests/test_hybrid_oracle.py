@@ -103,3 +103,41 @@ def test_a_prefix_has_the_logits_of_the_whole():
     tokens = torch.randint(0, 50, (11,), generator=torch.Generator().manual_seed(1))
     whole = O.forward(shape.to_config(), w, tokens, dtype=F64)
     assert torch.allclose(O.forward(shape.to_config(), w, tokens[:7], dtype=F64), whole[:7])
+
+
+def _planted():
+    """Mistakes that a kernel could make, planted in the plain implementation."""
+    norm, rot, att, wkv, lru, hyper, conv = (O.rms_norm, O.rotate_pairs, O.windowed_softmax_attention, O.wkv_recurrence, O.linear_recurrent_unit,
+                                             O.hyper_connection, O.causal_conv)
+    return {
+        "window one longer": ("windowed_softmax_attention", lambda q, k, v, s, w: att(q, k, v, s, w + 1)),
+        "window one shorter": ("windowed_softmax_attention", lambda q, k, v, s, w: att(q, k, v, s, w - 1)),
+        "rotation one position off on one side": ("rotate_pairs", lambda x, p, b: rot(x, p + (x.dim() == 3), b)),
+        "halves instead of pairs": ("rotate_pairs", lambda x, p, b: torch.cat([rot(x[..., ::2], p, b), x[..., 1::2]], -1)),
+        "no bonus": ("wkv_recurrence", lambda r, k, v, d, u: wkv(r, k, v, d, torch.zeros_like(u))),
+        "decay before the key": ("wkv_recurrence", lambda r, k, v, d, u: wkv(r, k, v, torch.cat([d[1:], d[-1:]]), u)),
+        "recurrence forgets at token 20": ("linear_recurrent_unit", lambda u, r, i, lam: torch.cat([lru(u[:20], r[:20], i[:20], lam), lru(u[20:], r[20:], i[20:], lam)])),
+        "wkv forgets at token 20": ("wkv_recurrence", lambda r, k, v, d, u: torch.cat([wkv(r[:20], k[:20], v[:20], d[:20], u), wkv(r[20:], k[20:], v[20:], d[20:], u)])),
+        "convolution forgets at token 20": ("causal_conv", lambda x, w, b: torch.cat([conv(x[:20], w, b), conv(x[20:], w, b)])),
+        "no shift": ("token_shift", lambda h, mu: h),
+        "mix transposed": ("hyper_connection", lambda x, i, m, o, f: hyper(x, i, m.T, o, f)),
+        "eps outside the root": ("rms_norm", lambda x, eps, weight=None: norm(x, 0.0, weight) if eps < 1e-4 else norm(x, eps / 2, weight)),
+    }
+
+
+@pytest.mark.parametrize("mistake", sorted(_planted()))
+def test_the_gpu_tests_sizes_show_a_planted_mistake(mistake, monkeypatch):
+    """Each mistake moves the logits of the GPU tests' models well beyond what those tests allow in fp32."""
+    from test_gpu_hybrid import SHAPES, TOL, error, tokens_of
+
+    worst = 0.0
+    for name in ("odd", "one_stream", "many_heads"):
+        shape = SHAPES[name]
+        w = synthetic.random_hybrid_weights(shape, 0)
+        tokens = torch.tensor(tokens_of(shape, 80))
+        want = O.forward(shape.to_config(), w, tokens, dtype=F64)
+        with monkeypatch.context() as m:
+            m.setattr(O, *_planted()[mistake])
+            got = O.forward(shape.to_config(), w, tokens, dtype=F64)
+        worst = max(worst, error(got, want))
+    assert worst > 20 * TOL[torch.float32], worst
