@@ -510,8 +510,9 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
     }
   } else if (op == OP_OUT_PROJECT) {
     // Eight lanes per row, one per stream: all streams of the row, the stream's column of the mix, its output weight and
-    // its weight in the next sublayer's input.  Only this instruction touches its rows of the streams in this stage, and
-    // their last writer arrived stages ago.
+    // its weight in the next sublayer's input.  The streams may be read before the wait: every output projection of a
+    // schedule deals the rows to the queues alike, so their last writer is this workgroup, and it has seen its stores
+    // acknowledged.
     const int r = o.start + (tid >> 3), q = tid & 7;
     if ((tid >> 3) < m.rows && q < S) {
       const bool down = o.sub == 1;

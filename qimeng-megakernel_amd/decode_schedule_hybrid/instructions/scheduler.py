@@ -3,7 +3,8 @@
 A layer is a chain of stages: input projections, the mixer's middle (recurrence; absorb, attend, value; wkv step), output
 projection, and for a feed-forward up/gate and down; the LM head ends the step.  Each stage's output rows are cut into
 blocks of equal size, about one per queue, and dealt to the queues from queue 0 on (the leaders of the per-XCD waits are
-the first eight queues, so they take part in every stage).  One tensor serves every position: the split of the visible
+the first eight queues, so they take part in every stage).  All output and down projections are cut alike: a queue owns its
+rows of the residual streams for the whole step, and the kernel relies on it.  One tensor serves every position: the split of the visible
 keys over the parts of opcode 4 is worked out on the device.
 """
 from __future__ import annotations

@@ -151,6 +151,18 @@ def test_schedule_covers_every_row_once(queues, pattern):
     assert all([i.wait_stage for i in q] == sorted(i.wait_stage for i in q) for q in lanes), "a queue runs its stages in order"
 
 
+@pytest.mark.parametrize("queues", [256, 24, 3])
+def test_a_queue_owns_its_rows_of_the_streams(queues):
+    owner: dict = {}
+    for q, column in enumerate(S.HybridScheduler(odd_shape(width=300, ff={"r": 36, "a": 20, "w": 52}), queues).instruction_queues()):
+        for ins in column:
+            if ins.opcode() == 7:
+                assert ins.count <= S.MAX_OUT_ROWS
+                for row in range(ins.start, ins.start + ins.count):
+                    assert owner.setdefault(row, q) == q
+    assert sorted(owner) == list(range(304))
+
+
 def test_one_leading_instruction_keeps_shared_rows():
     stages = S.HybridScheduler(odd_shape(pattern="aw"), 16).stages()
     assert sum(i.extra for s in stages for i in s if i.opcode() == 3) == 1
