@@ -11,6 +11,7 @@
 
 #include "qmk_hybrid_ops.h"
 #include "qmk_hybrid_prefill.h"
+#include "qmk_hybrid_plain.h"
 
 namespace qmk {
 namespace hybrid {
@@ -70,8 +71,11 @@ __global__ __launch_bounds__(kThreads, 1) void decode_megakernel_hybrid(const De
         case OP_WKV_STEP:
         case OP_OUT_PROJECT:
         case OP_UP_GATE:
-        case OP_LM_HEAD: ok = op_rows<T>(p, s, o); break;
-        case OP_LATENT_ATTEND: ok = op_latent_attend<T>(p, s, o); break;
+        case OP_LM_HEAD:
+        case OP_STATE_STEP:
+        case OP_JOIN: ok = op_rows<T>(p, s, o); break;
+        case OP_ATTEND: ok = op_attend<T>(p, s, o); break;
+        case OP_ATTEND_MERGE: ok = op_attend_merge(p, s, o); break;
         default:
           if (threadIdx.x == 0) report_error(counters_of(p), QMK_DEV_BAD_OPCODE, i, o.opcode, 0);
           ok = false;
@@ -158,7 +162,29 @@ inline size_t align_up(size_t n) { return (n + 255) & ~size_t(255); }
 inline bool m16(int v) { return v > 0 && v % 16 == 0; }
 inline int element(const QmkHybridArgs* a) { return a->dtype == QMK_HYBRID_F32 ? 4 : 2; }
 
-bool layer_ok(const QmkHybridArgs* a, const QmkHybridLayer& l) {
+// Entries of a plain residual: where they read x, and how a run's branches stand in the table.
+bool plain_ok(const QmkHybridArgs* a, int i) {
+  const QmkHybridLayer& l = a->layers[i];
+  const bool run = l.type >= QMK_MIXER_GLA && l.type <= QMK_MIXER_DELTA;
+  if (!run && l.type != QMK_ENTRY_JOIN && l.type != QMK_ENTRY_FINAL) return false;
+  if ((i + 1 == a->num_layers) != (l.type == QMK_ENTRY_FINAL)) return false;
+  if (l.branch < 0 || l.branches < 1 || l.branches > QMK_HYBRID_MAX_BRANCHES || l.branch >= l.branches || (!run && l.branches != 1)) return false;
+  if (i - l.branch < 0 || i - l.branch + l.branches > a->num_layers) return false;
+  for (int b = 0; b < l.branches; ++b) {
+    const QmkHybridLayer& other = a->layers[i - l.branch + b];
+    if (other.branch != b || other.branches != l.branches || (b > 0 && other.has_mlp)) return false;
+  }
+  if (l.x_from < -1 || l.x_from > 1 || l.x_to < 0 || l.x_to > 1 || l.x_from == l.x_to) return false;
+  if (l.prev < -1 || l.prev >= i || (l.prev >= 0 && (a->layers[l.prev].branch != 0 || a->layers[l.prev].type > QMK_MIXER_DELTA || l.x_from < 0))) return false;
+  return l.norm >= QMK_NORM_RMS && l.norm <= QMK_NORM_LAYER && l.proj_at >= 0 && l.proj_at % 16 == 0 && l.mix_at >= 0 && l.mix_at % 16 == 0 && l.ff_at >= 0 &&
+         l.ff_at % 16 == 0;
+}
+
+bool layer_ok(const QmkHybridArgs* a, int i) {
+  const QmkHybridLayer& l = a->layers[i];
+  if (a->streams == 0 ? !plain_ok(a, i) : l.type > QMK_MIXER_WKV) return false;
+  if (l.type == QMK_ENTRY_JOIN) return 2 * a->width <= kMaxK;
+  if (l.type == QMK_ENTRY_FINAL) return true;
   if (!m16(l.in_rows) || !m16(l.mix_width) || l.mix_width > kMaxK) return false;
   if (l.has_mlp && (!m16(l.ff) || l.ff > kMaxK)) return false;
   switch (l.type) {
@@ -173,6 +199,22 @@ bool layer_ok(const QmkHybridArgs* a, const QmkHybridLayer& l) {
     case QMK_MIXER_WKV:
       return l.heads > 0 && m16(l.head_dim) && l.head_dim <= kMaxHeadDim && l.head_dim_true > 0 && l.head_dim_true <= l.head_dim && m16(l.rank) &&
              l.rank <= kMaxK && l.mix_width == l.heads * l.head_dim && l.in_rows == 4 * l.mix_width + l.rank;
+    case QMK_MIXER_ATTENTION:
+      return l.heads > 0 && l.kv_heads > 0 && l.heads % l.kv_heads == 0 && m16(l.head_dim) && m16(l.v_dim) && l.v_dim <= 256 && l.rot_dim == 0 &&
+             l.rot_true >= 0 && l.rot_true % 2 == 0 && l.rot_true <= l.head_dim && l.q_stride == (l.head_dim + 31) / 32 * 32 && l.q_stride <= 256 &&
+             l.window > 0 && l.ring > 0 && l.mix_width == l.heads * l.v_dim &&
+             l.in_rows == l.heads * (l.q_stride + l.v_dim) + l.kv_heads * (l.head_dim + l.v_dim) &&
+             attend_floats(l.head_dim + l.v_dim, element(a)) <= kAttendFloats;
+    case QMK_MIXER_GLA:
+    case QMK_MIXER_DELTA: {
+      const bool delta = l.type == QMK_MIXER_DELTA;
+      if (l.heads < 1 || l.kv_heads < 1 || l.heads % l.kv_heads != 0 || !m16(l.head_dim) || l.head_dim > kMaxHeadDim || !m16(l.v_dim) || l.v_dim > kMaxHeadDim ||
+          l.v_true < 1 || l.v_true > l.v_dim || !m16(l.rank) || l.mix_width != l.heads * l.v_dim)
+        return false;
+      if (!delta) return l.kv_heads == l.heads && l.gate_rank == 0 && l.rank <= kMaxK && l.in_rows == 2 * l.heads * (l.head_dim + l.v_dim) + l.rank;
+      return m16(l.gate_rank) && l.rank + l.gate_rank <= kMaxK && l.taps >= 1 && l.taps <= kMaxTaps &&
+             l.in_rows == conv_channels(l) + l.rank + l.gate_rank + (l.heads + 15) / 16 * 16;
+    }
     default: return false;
   }
 }
@@ -181,15 +223,24 @@ int check_shape(const QmkHybridArgs* a) {
   if (a == nullptr || a->layers == nullptr) return QMK_ERR_NULL_ARG;
   if (a->struct_size != sizeof(QmkHybridArgs)) return QMK_ERR_ABI;
   if (a->dtype > QMK_HYBRID_F32) return QMK_ERR_MODEL;
-  if (a->num_layers < 1 || !m16(a->width) || a->width > kMaxK || a->width_true < 1 || a->width_true > a->width || a->streams < 1 ||
-      a->streams > kMaxStreams || a->vocab < 1 || !m16(a->vocab_rows) || a->vocab > a->vocab_rows || !(a->eps >= 0.f))
+  if (a->num_layers < 1 || !m16(a->width) || a->width > kMaxK || a->width_true < 1 || a->width_true > a->width || a->streams < 0 ||
+      a->streams > kMaxStreams || a->vocab < 1 || !m16(a->vocab_rows) || a->vocab > a->vocab_rows || !(a->eps >= 0.f) ||
+      !(a->logit_softcap >= 0.f))
     return QMK_ERR_SHAPE;
   for (int i = 0; i < a->num_layers; ++i)
-    if (!layer_ok(a, a->layers[i])) return QMK_ERR_SHAPE;
+    if (!layer_ok(a, i)) return QMK_ERR_SHAPE;
   return QMK_OK;
 }
 
 bool layer_pointers(const QmkHybridLayer& l) {
+  if (l.type == QMK_ENTRY_JOIN) return l.in_w != nullptr;
+  if (l.type == QMK_ENTRY_FINAL) return l.norm1 != nullptr;
+  if (l.type >= QMK_MIXER_GLA) {
+    bool ok = l.in_w && l.o_w && (l.branch > 0 || l.norm1) && (!l.has_mlp || (l.mlp_w && l.down_w)) && (l.branches > 1) == (l.out_norm != nullptr);
+    if (l.type == QMK_MIXER_ATTENTION) return ok && l.cache && ((l.rope_cos && l.rope_sin) || l.rot_true == 0);
+    ok = ok && l.mid_w && l.mid_b && l.vec0 && l.state;
+    return ok && (l.type == QMK_MIXER_GLA || (l.vec1 && l.vec2 && (l.shift || l.taps == 1)));
+  }
   bool ok = l.norm1 && l.in_w && l.mid_w && l.vec0;
   if (l.type == QMK_MIXER_LATENT) ok = ok && l.uk_w && l.uv_w && l.rope_cos && l.rope_sin && l.cache;
   else ok = ok && l.mid_b && l.vec1 && l.vec2 && l.state && (l.shift || (l.type == QMK_MIXER_RGLRU && l.taps == 1));
@@ -208,7 +259,7 @@ int check_launch(const QmkHybridArgs* a, int tokens) {
   for (int i = 0; i < a->num_layers; ++i) {
     const QmkHybridLayer& l = a->layers[i];
     // every key a query of the launch sees must still have its row when the launch's rows have been written
-    if (l.type == QMK_MIXER_LATENT && l.ring < std::min(a->position + tokens, l.window - 1 + tokens)) return QMK_ERR_SHAPE;
+    if ((l.type == QMK_MIXER_LATENT || l.type == QMK_MIXER_ATTENTION) && l.ring < std::min(a->position + tokens, l.window - 1 + tokens)) return QMK_ERR_SHAPE;
   }
   if (reinterpret_cast<uintptr_t>(a->workspace) % 256 != 0) return QMK_ERR_SHAPE;
   return QMK_OK;
@@ -227,14 +278,20 @@ struct Carver {
 
 struct DecodeBuffers {
   uint64_t* candidates;
-  float *u, *x, *proj, *mix, *absorbed, *part, *ml;
+  float *u, *x, *out, *proj, *mix, *absorbed, *part, *ml;
 };
 size_t decode_buffers(const QmkHybridArgs* a, void* base, DecodeBuffers* b) {
   size_t proj = 0, mix = 0, absorbed = 0, part = 0, ml = 0;
   for (int i = 0; i < a->num_layers; ++i) {
     const QmkHybridLayer& l = a->layers[i];
-    proj = std::max<size_t>(proj, l.in_rows);
-    mix = std::max<size_t>(mix, std::max(l.mix_width, l.has_mlp ? l.ff : 0));
+    if (l.type > QMK_MIXER_DELTA) continue;
+    proj = std::max<size_t>(proj, static_cast<size_t>(l.proj_at) + l.in_rows);
+    mix = std::max<size_t>(mix, std::max(static_cast<size_t>(l.mix_at) + l.mix_width, l.has_mlp ? static_cast<size_t>(l.ff_at) + l.ff : 0));
+    if (l.type == QMK_MIXER_ATTENTION) {
+      const size_t heads16 = (l.heads + 15) & ~15;
+      part = std::max(part, a->max_splits * heads16 * l.v_dim);
+      ml = std::max(ml, a->max_splits * heads16 * 2);
+    }
     if (l.type == QMK_MIXER_LATENT) {
       const size_t heads16 = (l.heads + 15) & ~15;
       absorbed = std::max<size_t>(absorbed, static_cast<size_t>(l.heads) * l.rank);
@@ -245,12 +302,67 @@ size_t decode_buffers(const QmkHybridArgs* a, void* base, DecodeBuffers* b) {
   Carver c{static_cast<char*>(base)};
   b->candidates = c.take<uint64_t>(kMaxQueues);
   b->u = c.take<float>(a->width);
-  b->x = c.take<float>(static_cast<size_t>(a->streams) * a->width);
+  b->x = c.take<float>(static_cast<size_t>(a->streams > 0 ? a->streams : 2) * a->width);
+  b->out = c.take<float>(a->streams > 0 ? 0 : static_cast<size_t>(QMK_HYBRID_MAX_BRANCHES + 1) * a->width);
   b->proj = c.take<float>(proj);
   b->mix = c.take<float>(mix);
   b->absorbed = c.take<float>(absorbed);
   b->part = c.take<float>(part);
   b->ml = c.take<float>(ml);
+  return c.used;
+}
+
+inline size_t values_cap(const QmkHybridArgs* a) { return (static_cast<size_t>(a->max_positions) + 31) & ~size_t(31); }
+
+template <class T>
+struct PlainBuffers {
+  float *x, *branch, *qkv, *decay, *beta, *o, *chunks;
+  T *h, *q, *low, *gate, *mix, *vt;
+};
+template <class T>
+size_t plain_buffers(const QmkHybridArgs* a, void* base, PlainBuffers<T>* b) {
+  const size_t P = a->portion_rows, D = a->width, chunks_of = (P + kChunkTokens - 1) / kChunkTokens;
+  size_t h = P * D, branch = 0, qkv = 0, decay = 0, beta = 0, o = 0, chunks = 0, q = 0, low = 0, gate = 0, mix = 0, vt = 0;
+  for (int i = 0; i < a->num_layers; ++i) {
+    const QmkHybridLayer& l = a->layers[i];
+    if (l.type == QMK_ENTRY_JOIN) h = std::max(h, 2 * P * D);
+    if (l.type > QMK_MIXER_DELTA) continue;
+    mix = std::max(mix, P * std::max<size_t>(l.mix_width, l.has_mlp ? l.ff : 0));
+    gate = std::max(gate, P * l.mix_width);
+    if (l.branches > 1) branch = std::max(branch, l.branches * P * D);
+    if (l.type == QMK_MIXER_ATTENTION) {
+      q = std::max(q, P * l.heads * l.q_stride);
+      vt = std::max(vt, values_cap(a) * l.kv_heads * l.v_dim);
+      continue;
+    }
+    decay = std::max(decay, P * l.heads * l.head_dim);
+    o = std::max(o, P * l.mix_width);
+    low = std::max(low, P * (l.rank + l.gate_rank));
+    chunks = std::max(chunks, chunks_of * l.heads * chunk_floats(l.head_dim));
+    if (l.type == QMK_MIXER_DELTA) {
+      q = std::max(q, P * conv_channels(l));
+      qkv = std::max(qkv, P * l.mix_width);
+      beta = std::max(beta, P * ((l.heads + 15) / 16 * 16));
+    } else {
+      qkv = std::max(qkv, P * (2 * l.heads * l.head_dim + l.mix_width));
+    }
+  }
+  Carver c{static_cast<char*>(base)};
+  PlainBuffers<T> local;
+  if (b == nullptr) b = &local;
+  b->x = c.take<float>(P * D);
+  b->branch = c.take<float>(branch);
+  b->qkv = c.take<float>(qkv);
+  b->decay = c.take<float>(decay);
+  b->beta = c.take<float>(beta);
+  b->o = c.take<float>(o);
+  b->chunks = c.take<float>(chunks);
+  b->h = c.take<T>(h);
+  b->q = c.take<T>(q);
+  b->low = c.take<T>(low);
+  b->gate = c.take<T>(gate);
+  b->mix = c.take<T>(mix);
+  b->vt = c.take<T>(vt);
   return c.used;
 }
 
@@ -263,6 +375,7 @@ struct PrefillBuffers {
 };
 template <class T>
 size_t prefill_buffers(const QmkHybridArgs* a, void* base, PrefillBuffers<T>* b) {
+  if (a->streams == 0) return plain_buffers<T>(a, base, nullptr);
   const size_t P = a->portion_rows, D = a->width;
   size_t h = P * D, fa = 0, fb = 0, raw = 0, p0 = 0, p1 = 0, p2 = 0, mix = 0, rows = 0, kn = 0, vt = 0;
   for (int i = 0; i < a->num_layers; ++i) {
@@ -327,14 +440,24 @@ void launch_gemm(const GemmArgs& g, hipStream_t st) {
   else hipLaunchKernelGGL((gemm<TA, TW, T, 64, 64>), grid(64, 64), block, 0, st, g);
 }
 
-template <class T, int QT, int VT>
-void launch_attention(const QmkHybridArgs* a, const QmkHybridLayer& l, const PrefillBuffers<T>& b, int first, int cap, hipStream_t st) {
-  hipLaunchKernelGGL((window_attention<T, QT, VT>), dim3((a->tokens + 63) / 64, l.heads), dim3(kPfThreads), 0, st, b.p0, b.kn, b.rows, b.vt, b.p1, l,
-                     first, a->position, a->tokens, cap, b.mix);
+// rows: where the rotated part of a latent attention's keys is, behind the latent.
+template <class T>
+void launch_attention(const QmkHybridArgs* a, const QmkHybridLayer& l, const T* q, Keys<T> keys, const T* rows, const T* vt, const T* gate, int first, int cap, T* out,
+                      hipStream_t st) {
+  auto launch = [&](auto kernel) {
+    hipLaunchKernelGGL(kernel, dim3((a->tokens + 63) / 64, l.heads), dim3(kPfThreads), 0, st, q, keys, rows, vt, gate, l, first, a->position, a->tokens, cap, out);
+  };
+  if (l.q_stride <= 128 && l.v_dim <= 64) launch(window_attention<T, 4, 4>);
+  else if (l.q_stride <= 192 && l.v_dim <= 128) launch(window_attention<T, 6, 8>);
+  else launch(window_attention<T, 8, 16>);
 }
 
 template <class T>
+int prefill_plain(const QmkHybridArgs* a);
+
+template <class T>
 int prefill(const QmkHybridArgs* a) {
+  if (a->streams == 0) return prefill_plain<T>(a);
   PrefillBuffers<T> b;
   if (prefill_buffers<T>(a, a->workspace, &b) > a->workspace_bytes) return QMK_ERR_SCRATCH;
   const hipStream_t st = static_cast<hipStream_t>(a->stream);
@@ -380,9 +503,8 @@ int prefill(const QmkHybridArgs* a) {
       GemmArgs v = gemm_args(nullptr, l.rank, nullptr, keys, l.rank, l, EPI_STORE);   // transposed: W_uv rows x keys
       v.a = l.uv_w; v.w = b.rows; v.ldw = width; v.M = l.heads * l.v_dim; v.out = b.vt; v.ldo = cap;
       launch_gemm<u16, T, T>(v, st);
-      if (l.q_stride <= 128 && l.v_dim <= 64) launch_attention<T, 4, 4>(a, l, b, first, cap, st);
-      else if (l.q_stride <= 192 && l.v_dim <= 128) launch_attention<T, 6, 8>(a, l, b, first, cap, st);
-      else launch_attention<T, 8, 16>(a, l, b, first, cap, st);
+      const Keys<T> expanded{b.kn, l.heads * l.head_dim, l.head_dim, 1};
+      launch_attention<T>(a, l, b.p0, expanded, b.rows, b.vt, b.p1, first, cap, b.mix, st);
     } else {
       const int N = W, n = l.head_dim;
       hipLaunchKernelGGL(shift_mix<T>, dim3(M), block, 0, st, b.u, l, a->slot, a->flip, M, P, D, a->width_true, a->eps, b.h);
@@ -417,6 +539,124 @@ int prefill(const QmkHybridArgs* a) {
     GemmArgs g = gemm_args(b.h, D, a->head, a->vocab_rows, D, a->layers[0], EPI_LOGITS);
     g.M = a->num_want; g.f0 = a->logits; g.ldo = a->vocab_rows;
     launch_gemm<T, u16, T>(g, st);
+  }
+  return hipGetLastError() == hipSuccess ? QMK_OK : QMK_ERR_LAUNCH;
+}
+
+// The recurrence of a gla or delta entry over the portion, from its projections to what its output projection reads.
+template <class T, bool DELTA>
+void run_chunks(const QmkHybridArgs* a, const ChunkArgs& g, hipStream_t st) {
+  const QmkHybridLayer& l = g.layer;
+  const int chunks = (g.M + kChunkTokens - 1) / kChunkTokens, tiles = l.head_dim / 16;
+  hipLaunchKernelGGL((chunk_prepare<T, DELTA>), dim3(chunks, l.heads), dim3(kPfThreads), 0, st, g);
+  const dim3 grid(l.heads, l.v_dim / 16), block(kChunkWaves * 64);
+  if (tiles <= kChunkWaves) hipLaunchKernelGGL((chunk_scan<1, DELTA>), grid, block, 0, st, g);
+  else if (tiles <= 2 * kChunkWaves) hipLaunchKernelGGL((chunk_scan<2, DELTA>), grid, block, 0, st, g);
+  else hipLaunchKernelGGL((chunk_scan<4, DELTA>), grid, block, 0, st, g);
+}
+
+template <class T>
+int prefill_plain(const QmkHybridArgs* a) {
+  PlainBuffers<T> b;
+  if (plain_buffers<T>(a, a->workspace, &b) > a->workspace_bytes) return QMK_ERR_SCRATCH;
+  const hipStream_t st = static_cast<hipStream_t>(a->stream);
+  const int M = a->tokens, D = a->width;
+  const size_t rows = static_cast<size_t>(a->portion_rows) * D;
+  const dim3 block(kPfThreads);
+  auto gemm_args = [&](const T* in, const u16* w, int N, int K, const QmkHybridLayer& l, int epi) {
+    GemmArgs g{};
+    g.a = in; g.lda = K; g.w = w; g.ldw = K; g.M = M; g.N = g.last_n = N; g.K = K; g.groups = 1;
+    g.layer = l; g.epi = epi; g.position = a->position; g.slot = a->slot; g.width = D; g.ldo = D;
+    g.logit_scale = a->logit_scale; g.logit_softcap = a->logit_softcap;
+    return g;
+  };
+  int runs_done = 0;
+  // x as entry l reads it: its norm (or [x; embedding]) -> h; `want`: of those rows alone, x stays.
+  auto residual = [&](const QmkHybridLayer& l, const int32_t* want, int count, bool added, float* dump) {
+    ResidualArgs g{};
+    g.x = b.x; g.table = a->embed; g.tokens = a->token_in; g.vocab = a->vocab; g.want = want; g.dump = dump;
+    g.weight = l.type == QMK_ENTRY_JOIN ? nullptr : l.norm1;
+    g.embed = l.x_from < 0; g.M = M; g.D = D; g.width = a->width_true; g.norm = l.norm; g.eps = a->eps;
+    if (added && l.prev >= 0 && a->layers[l.prev].branches == 2) {
+      const QmkHybridLayer* before = a->layers + l.prev;
+      g.a = b.branch; g.b = b.branch + rows; g.wa = before[0].out_norm; g.wb = before[1].out_norm; g.scale = before[0].out_scale;
+    }
+    hipLaunchKernelGGL(residual_rows<T>, dim3(count), block, 0, st, g, b.h);
+  };
+  auto dump_of = [&](const QmkHybridLayer& l) {   // where the run before this entry is asked for
+    return a->layer_out != nullptr && l.prev >= 0 ? a->layer_out + static_cast<size_t>(runs_done++) * M * D : nullptr;
+  };
+  for (int i = 0; i < a->num_layers; ++i) {
+    const QmkHybridLayer& l = a->layers[i];
+    const int W = l.mix_width;
+    if (l.type == QMK_ENTRY_FINAL) {
+      float* dump = dump_of(l);
+      if (dump != nullptr) residual(l, nullptr, M, true, dump);     // (and x is complete)
+      if (a->num_want > 0) {
+        residual(l, a->want, a->num_want, dump == nullptr, nullptr);
+        GemmArgs g = gemm_args(b.h, a->head, a->vocab_rows, D, l, EPI_CAPPED_LOGITS);
+        g.M = a->num_want; g.f0 = a->logits; g.ldo = a->vocab_rows;
+        launch_gemm<T, u16, T>(g, st);
+      }
+      break;
+    }
+    if (l.branch == 0) residual(l, nullptr, M, true, dump_of(l));
+    if (l.type == QMK_ENTRY_JOIN) {
+      GemmArgs g = gemm_args(b.h, l.in_w, D, 2 * D, l, EPI_LOGITS);
+      g.f0 = b.x;
+      launch_gemm<T, u16, T>(g, st);
+      continue;
+    }
+    if (l.type == QMK_MIXER_ATTENTION) {
+      GemmArgs g = gemm_args(b.h, l.in_w, l.in_rows, D, l, EPI_ATTENTION_IN);
+      g.out = b.q; g.out2 = b.gate;
+      launch_gemm<T, u16, T>(g, st);
+      const int row = l.head_dim + l.v_dim, pitch = l.kv_heads * row, keys = a->position + M, cap = static_cast<int>(values_cap(a));
+      const T* cache = static_cast<const T*>(l.cache) + static_cast<size_t>(a->slot) * l.ring * pitch;
+      hipLaunchKernelGGL(transpose_values<T>, dim3((keys + 63) / 64, (l.v_dim + 63) / 64, l.kv_heads), block, 0, st, cache, pitch, row, l.head_dim, l.v_dim, keys, cap, b.vt);
+      launch_attention<T>(a, l, b.q, Keys<T>{cache, pitch, row, l.heads / l.kv_heads}, nullptr, b.vt, b.gate, 0, cap, b.mix, st);
+    } else {
+      ChunkArgs c{};
+      c.layer = l; c.decay = b.decay; c.chunks = b.chunks; c.out = b.o; c.M = M; c.slot = a->slot; c.flip = a->flip;
+      if (l.type == QMK_MIXER_DELTA) {
+        const int channels = conv_channels(l), ranks = l.rank + l.gate_rank, beta_ld = (l.heads + 15) / 16 * 16;
+        GemmArgs g = gemm_args(b.h, l.in_w, l.in_rows, D, l, EPI_DELTA_IN);
+        g.out = b.q; g.out2 = b.low; g.f0 = b.beta; g.ldo = beta_ld;
+        launch_gemm<T, u16, T>(g, st);
+        GemmArgs e = gemm_args(b.low, l.mid_w, l.heads * (l.head_dim + l.v_dim), ranks, l, EPI_DELTA_MID);
+        e.f0 = b.decay; e.out = b.gate;
+        launch_gemm<T, u16, T>(e, st);
+        c.raw = b.q; c.beta = b.beta; c.beta_ld = beta_ld; c.values = b.qkv; c.value_ld = W;
+        run_chunks<T, true>(a, c, st);
+        if (l.taps > 1)
+          hipLaunchKernelGGL(keep_inputs<T>, dim3((channels + kPfThreads - 1) / kPfThreads), block, 0, st, b.q, l, channels, a->slot, a->flip, M);
+      } else {
+        const int keys = l.heads * l.head_dim;
+        GemmArgs g = gemm_args(b.h, l.in_w, l.in_rows, D, l, EPI_GLA_IN);
+        g.f0 = b.qkv; g.out = b.gate; g.out2 = b.low;
+        launch_gemm<T, u16, T>(g, st);
+        GemmArgs e = gemm_args(b.low, l.mid_w, keys, l.rank, l, EPI_GLA_MID);
+        e.f0 = b.decay; e.ldo = keys;
+        launch_gemm<T, u16, T>(e, st);
+        c.qkv = b.qkv; c.values = b.qkv; c.value_ld = 2 * keys + W; c.value_at = 2 * keys;
+        run_chunks<T, false>(a, c, st);
+      }
+      hipLaunchKernelGGL(state_out<T>, dim3((M * l.heads + 3) / 4), block, 0, st, b.o, b.gate, l, M, a->eps, b.mix);
+    }
+    GemmArgs o = gemm_args(b.mix, l.o_w, D, W, l, l.branches > 1 ? EPI_LOGITS : EPI_ADD);
+    o.f0 = l.branches > 1 ? b.branch + l.branch * rows : b.x;
+    launch_gemm<T, u16, T>(o, st);
+    if (l.branch + 1 == l.branches) {
+      const QmkHybridLayer& head = a->layers[i - l.branch];
+      if (head.has_mlp) {
+        GemmArgs g = gemm_args(b.h, head.mlp_w, 2 * head.ff, D, head, EPI_GEGLU);
+        g.out = b.mix;
+        launch_gemm<T, u16, T>(g, st);
+        GemmArgs d = gemm_args(b.mix, head.down_w, D, head.ff, head, EPI_ADD);
+        d.f0 = b.x;
+        launch_gemm<T, u16, T>(d, st);
+      }
+    }
   }
   return hipGetLastError() == hipSuccess ? QMK_OK : QMK_ERR_LAUNCH;
 }
@@ -464,10 +704,10 @@ extern "C" int qmk_hybrid_decode_step(const QmkHybridArgs* a) {
   DecodeParams p{};
   p.instructions = a->instructions; p.layers = a->layers_device; p.barriers = a->barriers; p.status = dev->status; p.timeline = a->timeline;
   p.candidates = b.candidates; p.embed = a->embed; p.head = a->head; p.final_norm = a->final_norm; p.token_in = a->token_in; p.token_out = a->token_out;
-  p.logits = a->logits; p.u = b.u; p.x = b.x; p.proj = b.proj; p.mix = b.mix; p.absorbed = b.absorbed; p.part = b.part; p.ml = b.ml;
+  p.logits = a->logits; p.u = b.u; p.x = b.x; p.out = b.out; p.proj = b.proj; p.mix = b.mix; p.absorbed = b.absorbed; p.part = b.part; p.ml = b.ml;
   p.num_insts = a->num_insts; p.num_layers = a->num_layers; p.groups = a->barrier_groups; p.width = a->width; p.width_true = a->width_true;
   p.streams = a->streams; p.vocab = a->vocab; p.vocab_rows = a->vocab_rows; p.slot = a->slot; p.position = a->position; p.flip = a->flip;
-  p.max_splits = a->max_splits; p.eps = a->eps; p.spin_limit = a->spin_limit != 0 ? a->spin_limit : kDefaultSpinLimit;
+  p.max_splits = a->max_splits; p.eps = a->eps; p.logit_scale = a->logit_scale; p.logit_softcap = a->logit_softcap; p.spin_limit = a->spin_limit != 0 ? a->spin_limit : kDefaultSpinLimit;
   const hipStream_t st = static_cast<hipStream_t>(a->stream);
   if (a->dtype == QMK_HYBRID_F32) hipLaunchKernelGGL(decode_megakernel_hybrid<float>, dim3(a->num_queues), dim3(kThreads), 0, st, p);
   else hipLaunchKernelGGL(decode_megakernel_hybrid<u16>, dim3(a->num_queues), dim3(kThreads), 0, st, p);

@@ -4,7 +4,9 @@
 // A step is a chain of stages; an instruction waits until every instruction of the stage before its own has arrived
 // (all-to-all edges on the per-XCD counters of qmk_device.h), so a buffer written in one stage may be overwritten two
 // stages later.  Activations between stages are fp32 and travel with device-coherent loads and stores; weights are
-// streamed once, bf16, and multiplied in fp32.  What does not depend on this step's earlier stages is asked for before an
+// streamed once, bf16, and multiplied in fp32.  On a plain residual no stage adds to it: the instructions that read it next
+// add what the layer run before has left (each for itself, one of them keeps the sum), so a norm over a branch's whole
+// output costs no stage of its own.  What does not depend on this step's earlier stages is asked for before an
 // instruction waits: its first weight rows, norm weights, recurrent states, old cache rows, the streams it will update.
 #pragma once
 
@@ -19,12 +21,15 @@ enum : int {
   OP_IN_PROJECT = 1,      // norm1 + the mixer's input projections, with what can be done per output behind them
   OP_LRU_STEP = 2,        // gates of one block + the recurrence of its channels
   OP_LATENT_ABSORB = 3,   // W_uk^T q per head; its leading instruction appends the cache row
-  OP_LATENT_ATTEND = 4,   // one part of the visible keys for 16 heads
+  OP_ATTEND = 4,          // one part of the visible keys for 16 heads
   OP_LATENT_VALUE = 5,    // merge of the parts, W_uv, output gate
   OP_WKV_STEP = 6,        // decay, recurrence, per-head norm and gate of one head
   OP_OUT_PROJECT = 7,     // output (sub 0) or down (sub 1) projection + all streams of the residual
   OP_UP_GATE = 8,         // norm2 + gate/up rows + gelu
   OP_LM_HEAD = 9,         // final norm + vocabulary rows
+  OP_STATE_STEP = 10,     // gla, delta: decay, recurrence, per-head norm and gate of one head
+  OP_ATTEND_MERGE = 11,   // merge of the parts of one head, output gate
+  OP_JOIN = 12,           // rows of [x; embedding] -> x
 };
 
 constexpr int kMaxStreams = QMK_HYBRID_MAX_STREAMS;
@@ -35,7 +40,8 @@ constexpr int kChunk = kWaveSize * 8;         // columns one wave covers with on
 constexpr int kMaxK = 24576;                  // longest activation vector
 constexpr int kAttendFloats = 33792;          // LDS of the attention op: query, key tile, scores
 constexpr int kMaxRank = 512;
-constexpr int kMaxHeadDim = 256;              // wkv
+constexpr int kMaxHeadDim = 256;              // wkv, gla, delta
+constexpr int kStateRows = 32;                // key rows of a head's state a thread holds in registers (gla, delta)
 constexpr int kMaxParts = 64;
 constexpr int kDepth = 8;                     // weight rows a wave keeps in flight and reduces together
 constexpr int kAhead = 2;                     // quads of a vector a thread holds in registers (4096 elements a workgroup)
@@ -56,7 +62,8 @@ struct DecodeParams {
   int64_t* token_out;
   float* logits;
   float* u;          // [D] input of the next sublayer before its norm
-  float* x;          // [streams][D]
+  float* x;          // [streams][D], plain: [2][D]
+  float* out;        // plain: [branches, feed-forward][D] what a layer run adds to x
   float* proj;       // outputs of OP_IN_PROJECT
   float* mix;        // what the output / down projection reads
   float* absorbed;   // [heads][rank]
@@ -69,7 +76,7 @@ struct DecodeParams {
   int32_t vocab, vocab_rows;
   int32_t slot, position, flip;
   int32_t max_splits;
-  float eps;
+  float eps, logit_scale, logit_softcap;
   uint32_t spin_limit;
 };
 
@@ -82,7 +89,7 @@ struct Smem {
     float attend[kAttendFloats];
   };
   float aux[3072];
-  float scratch[kWaves];
+  float scratch[3 * kWaves];
   int32_t inst[kInstWords];
   int32_t next_layer;
   int32_t ctl[4];          // [0] wait result, [1] last to retire
@@ -289,6 +296,24 @@ struct RowStream {
   }
 };
 
+// Three sums over the workgroup at once; `scratch` holds 3 kWaves floats.
+__device__ __forceinline__ void block_sum3(float (&v)[3], float* scratch) {
+  const int wave = threadIdx.x / kWaveSize;
+#pragma unroll
+  for (int i = 0; i < 3; ++i) v[i] = wave_sum(v[i]);
+  __syncthreads();
+  if ((threadIdx.x & (kWaveSize - 1)) == 0)
+#pragma unroll
+    for (int i = 0; i < 3; ++i) scratch[i * kWaves + wave] = v[i];
+  __syncthreads();
+#pragma unroll
+  for (int i = 0; i < 3; ++i) {
+    v[i] = 0.f;
+#pragma unroll
+    for (int w = 0; w < kWaves; ++w) v[i] += scratch[i * kWaves + w];
+  }
+}
+
 __device__ __forceinline__ void clear_part(Smem& s, int rows) {
   if (static_cast<int>(threadIdx.x) < rows)
 #pragma unroll
@@ -388,6 +413,138 @@ __device__ __forceinline__ void norm_to_xs(const DecodeParams& p, Smem& s, const
     xs_quad(s, i) = times(xs_quad(s, i), *reinterpret_cast<const float4*>(weight + i), inv);
 }
 
+__device__ __forceinline__ void st_shared_quad(float* to, float4 v) {
+  auto pair = [](float lo, float hi) { return (static_cast<uint64_t>(__float_as_uint(hi)) << 32) | __float_as_uint(lo); };
+  __hip_atomic_store(reinterpret_cast<uint64_t*>(to), pair(v.x, v.y), __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+  __hip_atomic_store(reinterpret_cast<uint64_t*>(to) + 1, pair(v.z, v.w), __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+}
+__device__ __forceinline__ float4 embed_quad(const u16* e, int i) {
+  const uint2 t = *reinterpret_cast<const uint2*>(e + i);
+  return make_float4(bf_lo(t.x), bf_hi(t.x), bf_lo(t.y), bf_hi(t.y));
+}
+__device__ __forceinline__ float4 plus(float4 a, float4 b) { return make_float4(a.x + b.x, a.y + b.y, a.z + b.z, a.w + b.w); }
+__device__ __forceinline__ float4 multiply_add(float4 a, float4 b, float c, float4 t) {   // a b c + t
+  return make_float4(fmaf(a.x * b.x, c, t.x), fmaf(a.y * b.y, c, t.y), fmaf(a.z * b.z, c, t.z), fmaf(a.w * b.w, c, t.w));
+}
+
+// The plain residual as a run (or the model's norm, or a loop's pass) reads it: the copy `x_from` plus what the run `prev`
+// left.  normed: its norm under `weight` -> xs (`ahead`: the thread's first weights); otherwise [x; embedding] -> xs.
+// keep: also leaves the sum in copy `x_to`.
+__device__ __forceinline__ void residual_to_xs(const DecodeParams& p, Smem& s, LayerRef& l, bool normed, bool keep, const float* weight, const float4 (&ahead)[kAhead]) {
+  const int D = p.width, tid = threadIdx.x;
+  const u16* e = p.embed;
+  if (l.x_from < 0 || !normed) e += static_cast<size_t>(token_of(p)) * D;
+  const float* x = l.x_from < 0 ? nullptr : p.x + static_cast<size_t>(l.x_from) * D;
+  const bool added = l.prev >= 0;
+  LayerRef& before = layer_of(p, added ? l.prev : 0);
+  const bool two = added && before.branches == 2, ff = added && before.has_mlp;
+  const float *wa = nullptr, *wb = nullptr;
+  if (two) {
+    wa = before.out_norm;
+    wb = layer_of(p, l.prev + 1).out_norm;
+  }
+  // x, feed-forward and a lone branch in `v`; two branches in `a` and `b`, their norm weights in `na` and `nb`
+  auto fetch = [&](int i, float4& v, float4& a, float4& b, float4& na, float4& nb) {
+    v = x == nullptr ? embed_quad(e, i) : ld_shared_quad(x + i);
+    if (!added) return;
+    a = ld_shared_quad(p.out + i);
+    if (two) {
+      b = ld_shared_quad(p.out + D + i);
+      na = *reinterpret_cast<const float4*>(wa + i);
+      nb = *reinterpret_cast<const float4*>(wb + i);
+    }
+    if (ff) v = plus(v, ld_shared_quad(p.out + static_cast<size_t>(QMK_HYBRID_MAX_BRANCHES) * D + i));
+    if (!two) v = plus(v, a);
+  };
+  float4 v[kAhead], a[kAhead], b[kAhead], na[kAhead], nb[kAhead];
+  const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f);
+  float sum[3] = {0.f, 0.f, 0.f};
+#pragma unroll
+  for (int j = 0; j < kAhead; ++j) {
+    const int i = (j * kThreads + tid) * 4;
+    v[j] = a[j] = b[j] = na[j] = nb[j] = zero;
+    if (i < D) fetch(i, v[j], a[j], b[j], na[j], nb[j]);
+  }
+  float sa = 0.f, sb = 0.f;
+  if (two) {
+#pragma unroll
+    for (int j = 0; j < kAhead; ++j) {
+      sum[0] = square(a[j], sum[0]);
+      sum[1] = square(b[j], sum[1]);
+    }
+#pragma unroll 1
+    for (int i = (kAhead * kThreads + tid) * 4; i < D; i += kThreads * 4) {
+      sum[0] = square(ld_shared_quad(p.out + i), sum[0]);
+      sum[1] = square(ld_shared_quad(p.out + D + i), sum[1]);
+    }
+    block_sum3(sum, s.scratch);
+    sa = before.out_scale / sqrtf(sum[0] / p.width_true + p.eps);
+    sb = before.out_scale / sqrtf(sum[1] / p.width_true + p.eps);
+#pragma unroll
+    for (int j = 0; j < kAhead; ++j) v[j] = multiply_add(b[j], nb[j], sb, multiply_add(a[j], na[j], sa, v[j]));
+  }
+  float* x_to = p.x + static_cast<size_t>(l.x_to) * D;
+  float total = 0.f;
+  auto take = [&](int i, float4 t) {
+    total += t.x + t.y + t.z + t.w;
+    if (keep) st_shared_quad(x_to + i, t);
+    if (!normed) {
+      xs_quad(s, i) = t;
+      xs_quad(s, D + i) = embed_quad(e, i);
+    }
+  };
+#pragma unroll
+  for (int j = 0; j < kAhead; ++j) {
+    const int i = (j * kThreads + tid) * 4;
+    if (i < D) take(i, v[j]);
+  }
+#pragma unroll 1
+  for (int i = (kAhead * kThreads + tid) * 4; i < D; i += kThreads * 4) {
+    float4 t = zero, ta = zero, tb = zero, ua = zero, ub = zero;
+    fetch(i, t, ta, tb, ua, ub);
+    if (two) t = multiply_add(tb, ub, sb, multiply_add(ta, ua, sa, t));
+    take(i, t);
+    if (normed) xs_quad(s, i) = t;
+  }
+  if (!normed) return;
+  const float mean = l.norm == QMK_NORM_LAYER ? block_sum(total, s.scratch) / p.width_true : 0.f;
+  auto centred = [&](int i, float4 t) {   // storage columns behind the true width stay zero
+    return make_float4(i < p.width_true ? t.x - mean : 0.f, i + 1 < p.width_true ? t.y - mean : 0.f, i + 2 < p.width_true ? t.z - mean : 0.f,
+                       i + 3 < p.width_true ? t.w - mean : 0.f);
+  };
+  float sq = 0.f;
+#pragma unroll
+  for (int j = 0; j < kAhead; ++j) {
+    v[j] = centred((j * kThreads + tid) * 4, v[j]);
+    sq = square(v[j], sq);
+  }
+#pragma unroll 1
+  for (int i = (kAhead * kThreads + tid) * 4; i < D; i += kThreads * 4) {
+    const float4 t = centred(i, xs_quad(s, i));
+    sq = square(t, sq);
+    xs_quad(s, i) = t;
+  }
+  const float inv = 1.f / sqrtf(block_sum(sq, s.scratch) / p.width_true + p.eps);
+#pragma unroll
+  for (int j = 0; j < kAhead; ++j) {
+    const int i = (j * kThreads + tid) * 4;
+    if (i < D) xs_quad(s, i) = times(v[j], ahead[j], inv);
+  }
+#pragma unroll 1
+  for (int i = (kAhead * kThreads + tid) * 4; i < D; i += kThreads * 4)
+    xs_quad(s, i) = times(xs_quad(s, i), *reinterpret_cast<const float4*>(weight + i), inv);
+}
+
+// log(1 + e^z) and the decays of the gated recurrences
+__device__ __forceinline__ float softplus(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+template <class Layer>
+__device__ __forceinline__ float delta_decay(const Layer& l, int head, float z) { return expf(l.vec1[head] * softplus(z)); }
+template <class Layer>
+__device__ __forceinline__ float gla_decay(const Layer& l, float z) { return expf(-softplus(-z) * l.decay_scale); }
+template <class Layer>
+__host__ __device__ constexpr int conv_channels(const Layer& l) { return 2 * l.kv_heads * l.head_dim + l.heads * l.v_dim; }
+__device__ __forceinline__ float soft_cap(float z, float cap) { return cap > 0.f ? cap * tanhf(z / cap) : z; }
+
 template <class Layer>
 __device__ __forceinline__ void rotate(const Layer& l, int position, int d, float& a, float& b) {
   if (d >= l.rot_true) return;
@@ -433,10 +590,16 @@ __device__ __forceinline__ bool rows_of(const DecodeParams& p, LayerRef& l, cons
       return l.type == QMK_MIXER_WKV && o.sub >= 0 && o.sub < l.heads && l.head_dim <= kMaxHeadDim &&
              set(l.mid_w, static_cast<long long>(o.sub) * l.head_dim, l.head_dim, l.rank);
     case OP_OUT_PROJECT:
-      if (o.count > kMaxOutRows) return false;
+      if (p.streams > 0 && o.count > kMaxOutRows) return false;
       if (o.sub == 1) return l.has_mlp && o.start + o.count <= D && set(l.down_w, o.start, o.count, l.ff);
       return o.start + o.count <= D && set(l.o_w, o.start, o.count, l.mix_width);
     case OP_UP_GATE: return l.has_mlp && o.start + o.count <= l.ff && set(l.mlp_w, 2LL * o.start, 2 * o.count, D);
+    case OP_STATE_STEP: {
+      if ((l.type != QMK_MIXER_GLA && l.type != QMK_MIXER_DELTA) || o.sub < 0 || o.sub >= l.heads || l.head_dim > kMaxHeadDim || l.v_dim > kMaxHeadDim) return false;
+      const int per = l.type == QMK_MIXER_DELTA ? l.head_dim + l.v_dim : l.head_dim;
+      return set(l.mid_w, static_cast<long long>(o.sub) * per, per, l.rank + l.gate_rank);
+    }
+    case OP_JOIN: return l.type == QMK_ENTRY_JOIN && o.start + o.count <= D && set(l.in_w, o.start, o.count, 2 * D);
     case OP_LM_HEAD: return o.start + o.count <= p.vocab_rows && set(p.head, o.start, o.count, D);
     default: return false;
   }
@@ -448,6 +611,8 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
   Rows m;
   if (!rows_of(p, l, o, m)) return bad_operand(p, o, o.start);
   const int tid = threadIdx.x, D = p.width, S = p.streams;
+  const bool plain = S == 0;
+  LayerRef& lead = layer_of(p, o.layer - l.branch);      // the run's first entry
   RowStream g;
   g.start(m.w, m.rows, m.columns);
   clear_part(s, m.rows);
@@ -457,27 +622,31 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
   const bool mine = tid < m.rows;
   const bool normed = op == OP_IN_PROJECT || op == OP_UP_GATE || op == OP_LM_HEAD;
   const bool wkv_in = op == OP_IN_PROJECT && l.type == QMK_MIXER_WKV;
-  const bool first = o.layer == 0 && (op == OP_IN_PROJECT || (op == OP_OUT_PROJECT && o.sub == 0));
-  const float* norm = op == OP_IN_PROJECT ? l.norm1 : op == OP_UP_GATE ? l.norm2 : p.final_norm;
-  const size_t shift_copy = l.type == QMK_MIXER_WKV ? static_cast<size_t>(D) : static_cast<size_t>(l.taps - 1) * l.mix_width;
+  const bool reads_x = plain && (normed || op == OP_JOIN);
+  const bool first = !plain && o.layer == 0 && (op == OP_IN_PROJECT || (op == OP_OUT_PROJECT && o.sub == 0));
+  const float* norm = plain ? lead.norm1 : op == OP_IN_PROJECT ? l.norm1 : op == OP_UP_GATE ? l.norm2 : p.final_norm;
+  const int channels = l.type == QMK_MIXER_DELTA ? conv_channels(l) : l.mix_width;
+  const size_t shift_copy = l.type == QMK_MIXER_WKV ? static_cast<size_t>(D) : static_cast<size_t>(l.taps - 1) * channels;
   const float* shift_old = l.shift + (static_cast<size_t>(p.slot) * 2 + p.flip) * shift_copy;
   float* shift_new = l.shift + (static_cast<size_t>(p.slot) * 2 + 1 - p.flip) * shift_copy;
   const float* mu = l.vec2 + static_cast<size_t>(o.sub) * D;
   float4 w0[kAhead], w1[kAhead], w2[kAhead];
   float a[kMaxStreams] = {}, b[kMaxStreams] = {};
   float out_weight = 0.f, next_weight = 0.f;
+  float held[kStateRows];      // OP_STATE_STEP: this thread's rows of the state
   float* state = nullptr;
   if (normed) {
     load_ahead(w0, norm, D);
     if (wkv_in) {
       load_ahead(w1, shift_old, D);
       load_ahead(w2, mu, D);
-    } else if (op == OP_IN_PROJECT && l.type == QMK_MIXER_RGLRU && mine) {
+    } else if (op == OP_IN_PROJECT && (l.type == QMK_MIXER_RGLRU || l.type == QMK_MIXER_DELTA) && mine) {
       // Everything of the convolution but the current input; the kept inputs move up by one.
-      const int W = l.mix_width, c = row - W;
-      a[0] = l.in_b[row];
-      if (c >= 0) {
-        float acc = l.vec1[c];
+      const bool lru = l.type == QMK_MIXER_RGLRU;
+      const int W = channels, c = lru ? row - W : row;
+      if (lru) a[0] = l.in_b[row];
+      if (c >= 0 && c < W) {
+        float acc = lru ? l.vec1[c] : 0.f;
 #pragma unroll 1
         for (int j = 0; j < l.taps - 1; ++j) {
           const float x = shift_old[static_cast<size_t>(j) * W + c];
@@ -508,7 +677,17 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
       const int at = o.sub * n + tid;
       w0[0] = make_float4(l.mid_b[at], l.vec1[at], l.vec0[at], 0.f);
     }
-  } else if (op == OP_OUT_PROJECT) {
+  } else if (op == OP_STATE_STEP) {
+    const int n = l.v_dim, groups = kThreads / n, e = tid % n, group = tid / n;
+    state = l.state + (static_cast<size_t>(p.slot) * l.heads + o.sub) * l.head_dim * n + e;
+#pragma unroll
+    for (int j = 0; j < kStateRows; ++j) {
+      const int i = group + j * groups;
+      held[j] = group < groups && i < l.head_dim ? state[static_cast<size_t>(i) * n] : 0.f;
+    }
+    if (tid < l.head_dim) a[0] = l.mid_b[o.sub * l.head_dim + tid];
+    if (tid < n) a[1] = l.vec0[tid];
+  } else if (op == OP_OUT_PROJECT && !plain) {
     // Eight lanes per row, one per stream: all streams of the row, the stream's column of the mix, its output weight and
     // its weight in the next sublayer's input.  The streams may be read before the wait: every output projection of a
     // schedule deals the rows to the queues alike, so their last writer is this workgroup, and it has seen its stores
@@ -533,7 +712,9 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
   if (!wait_stage(p, s, o)) return false;
 
   // The activation vector.
-  if (normed) {
+  if (reads_x) {
+    residual_to_xs(p, s, lead, normed, op == OP_IN_PROJECT && o.extra, norm, w0);
+  } else if (normed) {
     norm_to_xs(p, s, norm, w0, first, l.hc);
     if (wkv_in) {
       auto mix = [&](int i, float4 before, float4 m4) {
@@ -586,8 +767,38 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
     }
     if (in) s.xs[xs_at(tid)] = acc;
   } else {
-    const float* from = p.mix;
-    if (op == OP_LRU_STEP) {
+    const float* from = p.mix + (op == OP_OUT_PROJECT && o.sub == 1 ? l.ff_at : l.mix_at);
+    if (op == OP_STATE_STEP) {
+      // query, key (unit vectors for the delta rule) and value of the head
+      const bool delta = l.type == QMK_MIXER_DELTA;
+      const int n = l.v_dim, dim = l.head_dim, keys = l.kv_heads * dim, kv = o.sub / (l.heads / l.kv_heads);
+      const float* proj = p.proj + l.proj_at;
+      float q = 0.f, k = 0.f;
+      if (tid < dim) {
+        q = ld_shared_f32(proj + kv * dim + tid);
+        k = ld_shared_f32(proj + keys + kv * dim + tid);
+      }
+      if (tid < n) {
+        s.aux[2 * kMaxHeadDim + tid] = ld_shared_f32(proj + 2 * keys + o.sub * n + tid);
+        if (!delta) a[2] = ld_shared_f32(proj + 2 * keys + (l.heads + o.sub) * n + tid);      // the output gate
+      }
+      from = proj + 2 * keys + l.heads * n * (delta ? 1 : 2);
+      if (delta) a[3] = ld_shared_f32(from + l.rank + l.gate_rank + o.sub);      // beta
+      if (!delta) q *= l.q_scale;                       // (the projection is left unscaled)
+      float dots[3] = {q * q, k * k, q * k};
+      block_sum3(dots, s.scratch);
+      if (delta) {
+        const float iq = l.q_scale / sqrtf(dots[0] + 1e-6f), ik = 1.f / sqrtf(dots[1] + 1e-6f);
+        q *= iq;
+        k *= ik;
+        dots[2] *= iq * ik;
+      }
+      a[4] = dots[2];
+      if (tid < dim) {
+        s.aux[tid] = q;
+        s.aux[kMaxHeadDim + tid] = k;
+      }
+    } else if (op == OP_LRU_STEP) {
       if (mine && !(tid & 1)) a[3] = ld_shared_f32(p.proj + o.sub * l.block_dim + o.start + (tid >> 1));
       from = p.proj + l.mix_width + o.sub * l.block_dim;
     } else if (op == OP_LATENT_ABSORB) {
@@ -613,9 +824,13 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
   stamp(p, s, 2);
 
   // What happens to the rows' sums; a pair of rows is a pair of lanes.
-  float t = mine && op != OP_OUT_PROJECT ? row_total(s, tid) : 0.f;
+  float t = mine && (plain || op != OP_OUT_PROJECT) ? row_total(s, tid) : 0.f;
   static_assert(kMaxRows <= kThreads && kMaxStreams == 8, "one row per thread, eight values ahead");
-  if (op == OP_OUT_PROJECT) {
+  if (op == OP_JOIN) {
+    if (mine) st_shared_f32(p.x + static_cast<size_t>(l.x_to) * D + row, t);
+  } else if (op == OP_OUT_PROJECT && plain) {
+    if (mine) st_shared_f32(p.out + static_cast<size_t>(o.sub == 1 ? QMK_HYBRID_MAX_BRANCHES : l.branch) * D + row, t);
+  } else if (op == OP_OUT_PROJECT) {
     const int r = tid >> 3, q = tid & 7;
     if (r < m.rows) {      // whole groups of eight lanes
       float now = out_weight * row_total(s, r);
@@ -627,7 +842,7 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
     }
   } else if (op == OP_UP_GATE) {
     const float up = dpp_f32<kDppQuadXor1>(0.f, t);
-    if (mine && !(tid & 1)) st_shared_f32(p.mix + o.start + (tid >> 1), gelu_tanh(t) * up);
+    if (mine && !(tid & 1)) st_shared_f32(p.mix + l.ff_at + o.start + (tid >> 1), (l.act == QMK_ACT_SILU ? t * sigmoid(t) : gelu_tanh(t)) * up);
   } else if (op == OP_IN_PROJECT) {
     const float pair = dpp_f32<kDppQuadXor1>(0.f, t);
     if (mine) {
@@ -652,6 +867,26 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
           const float c = l.rope_cos[at], sn = l.rope_sin[at];
           t = t * c + ((tid & 1) ? pair * sn : -(pair * sn));
         }
+      } else if (l.type == QMK_MIXER_ATTENTION) {
+        const int q_rows = l.heads * l.q_stride, k_rows = l.kv_heads * l.head_dim, v_rows = l.kv_heads * l.v_dim;
+        const int d = row < q_rows ? row % l.q_stride : row < q_rows + k_rows ? (row - q_rows) % l.head_dim : l.rot_true;
+        if (d < l.rot_true) {
+          const size_t at = static_cast<size_t>(p.position) * (l.rot_true / 2) + (d >> 1);
+          const float c = l.rope_cos[at], sn = l.rope_sin[at];
+          t = t * c + ((tid & 1) ? pair * sn : -(pair * sn));
+        }
+        if (row >= q_rows + k_rows + v_rows) gate = 1;
+      } else if (l.type == QMK_MIXER_DELTA) {
+        if (row < channels) {
+          if (l.taps > 1) shift_new[static_cast<size_t>(l.taps - 2) * channels + row] = t;
+          t = fmaf(a[2], t, a[1]);
+          gate = 2;
+        } else if (row >= channels + l.rank + l.gate_rank) {
+          gate = 1;
+        }
+      } else if (l.type == QMK_MIXER_GLA) {
+        const int from = 2 * l.heads * l.head_dim + l.heads * l.v_dim;
+        if (row >= from && row < from + l.heads * l.v_dim) gate = 2;
       } else if (row >= 4 * W) {
         t = tanhf(t);
       } else if (row >= 3 * W) {
@@ -662,7 +897,7 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
         const float sg = sigmoid(z);
         t = gate == 1 ? sg : t * sg;
       }
-      st_shared_f32(p.proj + row, t);
+      st_shared_f32(p.proj + l.proj_at + row, t);
     }
   } else if (op == OP_LRU_STEP) {
     const float gate = sigmoid(t + a[0]), in_gate = dpp_f32<kDppQuadXor1>(0.f, gate);
@@ -728,7 +963,58 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
     const float sq = block_sum(val * val, s.scratch);   // storage columns behind the true head size hold zeros
     const float inv = 1.f / sqrtf(sq / l.head_dim_true + p.eps);
     if (mine) st_shared_f32(p.mix + o.sub * n + tid, val * inv * w0[0].z * w0[0].w);
+  } else if (op == OP_STATE_STEP) {
+    // S <- decay S, u = beta (v - S^T k), S <- S + k u^T, o = S^T q, with S^T k and S^T q taken together:
+    // o = (decay S)^T q + (q . k) u.  Without the delta rule u = v.
+    const bool delta = l.type == QMK_MIXER_DELTA;
+    const int n = l.v_dim, dim = l.head_dim, groups = kThreads / n, e = tid % n, group = tid / n;
+    float *q = s.aux, *k = q + kMaxHeadDim, *v = k + kMaxHeadDim, *w = v + kMaxHeadDim, *gate = w + kMaxHeadDim;
+    if (tid < dim) w[tid] = delta ? delta_decay(l, o.sub, t + a[0]) : gla_decay(l, t + a[0]);
+    else if (mine) gate[tid - dim] = sigmoid(t);
+    __syncthreads();
+    float ak = 0.f, aq = 0.f;
+    if (group < groups) {
+#pragma unroll
+      for (int j = 0; j < kStateRows; ++j) {
+        const int i = group + j * groups;
+        if (i < dim) {
+          held[j] *= w[i];
+          ak = fmaf(k[i], held[j], ak);
+          aq = fmaf(q[i], held[j], aq);
+        }
+      }
+#pragma unroll 1
+      for (int i = group + kStateRows * groups; i < dim; i += groups) {
+        const float h = w[i] * state[static_cast<size_t>(i) * n];
+        ak = fmaf(k[i], h, ak);
+        aq = fmaf(q[i], h, aq);
+      }
+      s.xs[group * n + e] = ak;
+      s.xs[(groups + group) * n + e] = aq;
+    }
+    __syncthreads();
+    ak = aq = 0.f;
+#pragma unroll 4
+    for (int i = 0; i < groups; ++i) {
+      ak += s.xs[i * n + e];
+      aq += s.xs[(groups + i) * n + e];
+    }
+    const float u = delta ? a[3] * (v[e] - ak) : v[e];
+    if (group < groups) {
+#pragma unroll
+      for (int j = 0; j < kStateRows; ++j) {
+        const int i = group + j * groups;
+        if (i < dim) state[static_cast<size_t>(i) * n] = fmaf(k[i], u, held[j]);
+      }
+#pragma unroll 1
+      for (int i = group + kStateRows * groups; i < dim; i += groups)
+        state[static_cast<size_t>(i) * n] = fmaf(k[i], u, w[i] * state[static_cast<size_t>(i) * n]);
+    }
+    const float val = tid < n ? fmaf(a[4], u, aq) : 0.f;
+    const float inv = 1.f / sqrtf(block_sum(val * val, s.scratch) / l.v_true + p.eps);
+    if (tid < n) st_shared_f32(p.mix + l.mix_at + o.sub * n + tid, val * inv * a[1] * (delta ? gate[tid] : a[2]));
   } else {   // OP_LM_HEAD
+    if (plain) t = soft_cap(t * p.logit_scale, p.logit_softcap);
     if (mine) p.logits[row] = t;
     const bool real = mine && row < p.vocab;
     const float top = block_max(real ? t : -INFINITY, s.scratch);
@@ -793,27 +1079,35 @@ __device__ __forceinline__ f32x4 mma(const Frag<float>& a, const Frag<u16>& b, f
 
 constexpr float kLog2e = 1.4426950408889634f;
 
-// Keys of one tile of OP_LATENT_ATTEND, and the LDS floats it needs for this cache row width (host and device).
+// Keys of one tile of OP_ATTEND, and the LDS floats it needs for this cache row width (host and device).
 __host__ __device__ constexpr int attend_keys(int element_bytes) { return element_bytes == 2 ? 64 : 32; }
 __host__ __device__ constexpr int attend_floats(int row_elements, int element_bytes) {
   const int stride = (row_elements + 31) / 32 * 32 + 8, keys = attend_keys(element_bytes), slices = kWaves / (keys / 16);
   return (16 + keys) * stride * element_bytes / 4 + slices * keys * 16 + keys * 16 + 16 * (keys + 8) + 16;
 }
 
-// Part `start` of `count` of the visible keys, heads [16 sub, 16 sub + 16).  Scores: matrix tiles of 16 keys x 16 heads,
-// the row's columns split over the waves of a tile; then the weights and the running sums of weight x latent, of which an
-// instruction keeps columns [128 extra, 128 extra + 128), sixteen a wave.
+// Part `start` of `count` of the visible keys, sixteen heads.  Scores: matrix tiles of 16 keys x 16 heads, the row's columns
+// split over the waves of a tile; then the weights and the running sums of weight x value, of which an instruction keeps
+// columns [128 extra, 128 extra + 128), sixteen a wave.
+// Latent: heads [16 sub, 16 sub + 16), a row is [latent | rotated key], the latent is the value.  Attention: the heads of key
+// head g = sub / b, sixteen of them from 16 (sub % b) on, b = ceil(heads per key head / 16); a row is g's [key | value], and
+// the step's own row comes from the projections (one instruction per key head puts it into the cache).
 template <class T>
-__device__ __forceinline__ bool op_latent_attend(const DecodeParams& p, Smem& s, const Op& o) {
+__device__ __forceinline__ bool op_attend(const DecodeParams& p, Smem& s, const Op& o) {
   constexpr int kKeys = attend_keys(sizeof(T)), kTiles = kKeys / 16, kSlices = kWaves / kTiles, kPer = kKeys * 16 / kThreads, kSp = kKeys + 8;
   constexpr int kUnit = 16 / sizeof(T);
   LayerRef& l = layer_of(p, o.layer);
   const int heads16 = (l.heads + 15) & ~15;
-  if (l.type != QMK_MIXER_LATENT || o.sub < 0 || o.sub * 16 >= l.heads || o.start < 0 || o.count <= 0 || o.count > p.max_splits || o.start >= o.count ||
-      o.extra < 0 || o.extra * 16 * kWaves >= l.rank)
+  const bool latent = l.type == QMK_MIXER_LATENT;
+  if ((!latent && l.type != QMK_MIXER_ATTENTION) || o.sub < 0 || o.start < 0 || o.count <= 0 || o.count > p.max_splits || o.start >= o.count || o.extra < 0)
     return bad_operand(p, o, o.start);
+  const int group = latent ? l.heads : l.heads / l.kv_heads, blocks = (group + 15) / 16, kv = o.sub / blocks, block = o.sub % blocks;
+  const int values = latent ? l.rank : l.v_dim, value_at = latent ? 0 : l.head_dim;      // columns of a row that are its value
+  const int head0 = kv * group + block * 16, heads = min(16, group - block * 16);
+  if (kv >= (latent ? 1 : l.kv_heads) || o.extra * 16 * kWaves >= values) return bad_operand(p, o, o.sub);
   const int tid = threadIdx.x, lane = tid & (kWaveSize - 1), wave = __builtin_amdgcn_readfirstlane(tid / kWaveSize);
-  const int width = l.rank + l.rot_dim, width32 = (width + 31) & ~31, stride = width32 + 8;
+  const int width = latent ? l.rank + l.rot_dim : l.head_dim + l.v_dim, width32 = (width + 31) & ~31, stride = width32 + 8;
+  const int pitch = latent ? width : l.kv_heads * width;      // elements between cache rows
   T* sq = reinterpret_cast<T*>(s.attend);
   T* sc = sq + 16 * stride;
   float* sred = reinterpret_cast<float*>(sc + kKeys * stride);   // [slice][key][16]
@@ -826,7 +1120,7 @@ __device__ __forceinline__ bool op_latent_attend(const DecodeParams& p, Smem& s,
   const int lo = first + o.start * per, hi = min(lo + per, p.position + 1);
   const int units = width32 / kUnit;
   const int rows = l.ring, offset = p.slot * rows;
-  const T* cache = static_cast<const T*>(l.cache);
+  T* cache = static_cast<T*>(l.cache) + kv * width;
   // Rows base .. base + kKeys - 1 -> sc, but for the row another workgroup of this launch appends.  (A part is never
   // longer than the ring, so a position wraps at most once.)
   auto load_tile = [&](int base) {
@@ -842,7 +1136,7 @@ __device__ __forceinline__ bool op_latent_attend(const DecodeParams& p, Smem& s,
           const int r = r0 + j * kWaves, at = at0 + r >= rows ? at0 + r - rows : at0 + r;
           v[j] = v4u{0u, 0u, 0u, 0u};
           if (base + r < hi && base + r != p.position && c * kUnit < width)
-            v[j] = *reinterpret_cast<const v4u*>(cache + static_cast<size_t>(offset + at) * width + c * kUnit);
+            v[j] = *reinterpret_cast<const v4u*>(cache + static_cast<size_t>(offset + at) * pitch + c * kUnit);
         }
 #pragma unroll
         for (int j = 0; j < kBatch; ++j) *reinterpret_cast<v4u*>(sc + (r0 + j * kWaves) * stride + c * kUnit) = v[j];
@@ -852,7 +1146,23 @@ __device__ __forceinline__ bool op_latent_attend(const DecodeParams& p, Smem& s,
   // The appended row, where this part holds it (it is then the part's last).
   auto load_appended = [&](int base) {
     if (p.position >= hi || p.position < base || p.position >= base + kKeys) return;
-    const T* row = cache + static_cast<size_t>(offset + p.position % rows) * width;
+    T* row = cache + static_cast<size_t>(offset + p.position % rows) * pitch;
+    if (!latent) {   // neighbouring elements, both of the key or both of the value
+      const float* from = p.proj + l.proj_at + l.heads * l.q_stride;
+      const bool put = block == 0 && o.extra == 0;
+#pragma unroll 1
+      for (int c = tid * 2; c < width; c += kThreads * 2) {
+        const uint64_t v = ld_shared64(from + (c < l.head_dim ? kv * l.head_dim + c : l.kv_heads * l.head_dim + kv * l.v_dim + c - l.head_dim));
+        T* at = sc + (p.position - base) * stride + c;
+        at[0] = from_f32<T>(__uint_as_float(static_cast<uint32_t>(v)));
+        at[1] = from_f32<T>(__uint_as_float(static_cast<uint32_t>(v >> 32)));
+        if (put) {
+          row[c] = at[0];
+          row[c + 1] = at[1];
+        }
+      }
+      return;
+    }
 #pragma unroll 1
     for (int c = tid; c * kUnit < width; c += kThreads) *reinterpret_cast<v4u*>(sc + (p.position - base) * stride + c * kUnit) = ld_shared128(row + c * kUnit);
   };
@@ -860,14 +1170,14 @@ __device__ __forceinline__ bool op_latent_attend(const DecodeParams& p, Smem& s,
   stamp(p, s, 0);
   if (!wait_stage(p, s, o)) return false;
   if (lo < hi) {
-    const int heads = min(16, l.heads - o.sub * 16);
 #pragma unroll 1
     for (int k = tid * 2; k < width32; k += kThreads * 2) {
       uint64_t v[16];
-      const float* from = k < l.rank ? p.absorbed + o.sub * 16 * l.rank + k : p.proj + o.sub * 16 * l.q_stride + l.head_dim + k - l.rank;
-      const int pitch = k < l.rank ? l.rank : l.q_stride;
+      const float* from = !latent ? p.proj + l.proj_at + head0 * l.q_stride + k
+                          : k < l.rank ? p.absorbed + head0 * l.rank + k : p.proj + head0 * l.q_stride + l.head_dim + k - l.rank;
+      const int step = latent && k < l.rank ? l.rank : l.q_stride, end = latent ? width : l.q_stride;
 #pragma unroll
-      for (int h = 0; h < 16; ++h) v[h] = h < heads && k < width ? ld_shared64(from + h * pitch) : 0;
+      for (int h = 0; h < 16; ++h) v[h] = h < heads && k < end ? ld_shared64(from + h * step) : 0;
 #pragma unroll
       for (int h = 0; h < 16; ++h) {
         sq[h * stride + k] = from_f32<T>(__uint_as_float(static_cast<uint32_t>(v[h])));
@@ -883,7 +1193,7 @@ __device__ __forceinline__ bool op_latent_attend(const DecodeParams& p, Smem& s,
   float m = -INFINITY, lsum = 0.f;
   f32x4 acc = {};
   const int column0 = (o.extra * kWaves + wave) * 16;      // this wave's sixteen columns of the latent
-  const bool columns = column0 < l.rank;
+  const bool columns = column0 < values;
 #pragma unroll 1
   for (int base = lo; base < hi; base += kKeys) {
     if (base != lo) {
@@ -893,7 +1203,7 @@ __device__ __forceinline__ bool op_latent_attend(const DecodeParams& p, Smem& s,
     }
     __syncthreads();
     {
-      const int tile = wave % kTiles, slice = wave / kTiles, steps = width32 / 32;
+      const int tile = wave % kTiles, slice = wave / kTiles, steps = (latent ? width32 : l.q_stride) / 32;
       f32x4 d = {};
       for (int k = slice; k < steps; k += kSlices)
         d = mma(load_frag(sc + (tile * 16 + (lane & 15)) * stride + k * 32 + (lane >> 4) * 8),
@@ -941,7 +1251,7 @@ __device__ __forceinline__ bool op_latent_attend(const DecodeParams& p, Smem& s,
       for (int kk = 0; kk < kKeys / 32; ++kk) {
         Frag<T> cf;
 #pragma unroll
-        for (int j = 0; j < 8; ++j) cf.set(j, sc[(kk * 32 + (lane >> 4) * 8 + j) * stride + column0 + (lane & 15)]);
+        for (int j = 0; j < 8; ++j) cf.set(j, sc[(kk * 32 + (lane >> 4) * 8 + j) * stride + value_at + column0 + (lane & 15)]);
         acc = mma(cf, load_frag(sp + (lane & 15) * kSp + kk * 32 + (lane >> 4) * 8), acc);
       }
     }
@@ -953,22 +1263,72 @@ __device__ __forceinline__ bool op_latent_attend(const DecodeParams& p, Smem& s,
   lsum += __shfl_xor(lsum, 32);
   if (lane < 16) ss[wave * 16 + head] = lsum;
   __syncthreads();
-  float* ml = p.ml + (static_cast<size_t>(o.start) * heads16 + o.sub * 16) * 2;
-  if (key0 == 0 && o.extra == 0) {
+  float* ml = p.ml + (static_cast<size_t>(o.start) * heads16 + head0) * 2;
+  if (key0 == 0 && o.extra == 0 && (latent || head < heads)) {
     float t = 0.f;
 #pragma unroll
     for (int k = 0; k < kWaves; ++k) t += ss[k * 16 + head];
     st_shared_f32(ml + head * 2, m);
     st_shared_f32(ml + head * 2 + 1, t);
   }
-  if (columns) {
-    uint64_t* at = reinterpret_cast<uint64_t*>(p.part + (static_cast<size_t>(o.start) * heads16 + o.sub * 16 + (lane & 15)) * l.rank + column0 + (lane >> 4) * 4);
+  if (columns && (latent || (lane & 15) < heads)) {
+    uint64_t* at = reinterpret_cast<uint64_t*>(p.part + (static_cast<size_t>(o.start) * heads16 + head0 + (lane & 15)) * values + column0 + (lane >> 4) * 4);
 #pragma unroll
     for (int i = 0; i < 2; ++i)
       __hip_atomic_store(at + i, (static_cast<uint64_t>(__float_as_uint(acc[2 * i + 1])) << 32) | __float_as_uint(acc[2 * i]), __ATOMIC_RELAXED,
                          __HIP_MEMORY_SCOPE_AGENT);
   }
   stamp(p, s, 3);
+  arrive_stage(p, o);
+  return true;
+}
+
+// The parts of one head put together, times its output gate.
+__device__ __forceinline__ bool op_attend_merge(const DecodeParams& p, Smem& s, const Op& o) {
+  LayerRef& l = layer_of(p, o.layer);
+  if (l.type != QMK_MIXER_ATTENTION || o.sub < 0 || o.sub >= l.heads || o.count <= 0 || o.count > p.max_splits || o.count > kMaxParts)
+    return bad_operand(p, o, o.sub);
+  const int tid = threadIdx.x, heads16 = (l.heads + 15) & ~15, parts = o.count, n = l.v_dim, groups = kThreads / n, e = tid % n, group = tid / n;
+  if (!wait_stage(p, s, o)) return false;
+  if (tid < parts) {
+    const uint64_t ml = ld_shared64(p.ml + (static_cast<size_t>(tid) * heads16 + o.sub) * 2);
+    s.aux[tid] = __uint_as_float(static_cast<uint32_t>(ml));
+    s.aux[kMaxParts + tid] = __uint_as_float(static_cast<uint32_t>(ml >> 32));
+  }
+  const float gate = tid < n ? ld_shared_f32(p.proj + l.proj_at + l.heads * l.q_stride + l.kv_heads * (l.head_dim + n) + o.sub * n + tid) : 0.f;
+  constexpr int kBatch = 8;
+  float v[kBatch];
+  const float* column = p.part + static_cast<size_t>(o.sub) * n + e;
+  auto request = [&](int base) {
+#pragma unroll
+    for (int j = 0; j < kBatch; ++j) v[j] = ld_shared_f32(column + static_cast<size_t>(min(base + j * groups, parts - 1)) * heads16 * n);
+  };
+  request(group);
+  __syncthreads();
+  if (tid < kWaveSize) {   // weights of the parts
+    const float mx = tid < parts ? s.aux[tid] : -INFINITY, top = wave_max(mx);
+    const float w = exp2_fast(mx - top), sum = wave_sum(tid < parts ? w * s.aux[kMaxParts + tid] : 0.f);
+    s.aux[tid] = tid < parts ? w / sum : 0.f;
+  }
+  __syncthreads();
+  float acc = 0.f;
+  if (group < groups) {
+#pragma unroll 1
+    for (int base = group; base < parts; base += kBatch * groups) {
+      if (base != group) request(base);
+#pragma unroll
+      for (int j = 0; j < kBatch; ++j)
+        if (base + j * groups < parts) acc = fmaf(s.aux[base + j * groups], v[j], acc);
+    }
+    s.xs[group * n + e] = acc;
+  }
+  __syncthreads();
+  if (tid < n) {
+    acc = 0.f;
+#pragma unroll 4
+    for (int i = 0; i < groups; ++i) acc += s.xs[i * n + tid];
+    st_shared_f32(p.mix + l.mix_at + o.sub * n + tid, acc * gate);
+  }
   arrive_stage(p, o);
   return true;
 }

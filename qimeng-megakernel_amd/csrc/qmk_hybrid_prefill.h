@@ -22,6 +22,13 @@ enum : int {
   EPI_WKV_IN,           // r, k, v fp32; silu gate; tanh
   EPI_WKV_DECAY,        // exp(-exp(. + w0))
   EPI_LOGITS,
+  EPI_CAPPED_LOGITS,    // logits times a constant, softly capped
+  EPI_ADD,              // onto the fp32 residual
+  EPI_ATTENTION_IN,     // rotation of q and k, k and v into the cache, sigmoid of the gate
+  EPI_DELTA_IN,         // raw q, k, v; raw ranks; sigmoid of the step sizes
+  EPI_DELTA_MID,        // decays and output gate
+  EPI_GLA_IN,           // q, k, v fp32; silu gate; raw rank
+  EPI_GLA_MID,          // decays
 };
 
 struct GemmArgs {
@@ -37,7 +44,8 @@ struct GemmArgs {
   const void* src;
   int ldo;
   QmkHybridLayer layer;
-  int down, first, position, streams, width, rows_cap;
+  int down, first, position, streams, width, rows_cap, slot;
+  float logit_scale, logit_softcap;
   const float* next;
 };
 
@@ -143,7 +151,8 @@ __device__ __forceinline__ void epilogue(const GemmArgs& g, int group, int m, in
     }
     case EPI_GEGLU: {
       T* o = static_cast<T*>(g.out) + static_cast<size_t>(m) * l.ff + n / 2;
-      const float a = gelu_tanh(v[0]) * v[1], b = gelu_tanh(v[2]) * v[3];
+      const bool silu = l.act == QMK_ACT_SILU;
+      const float a = (silu ? v[0] * sigmoid(v[0]) : gelu_tanh(v[0])) * v[1], b = (silu ? v[2] * sigmoid(v[2]) : gelu_tanh(v[2])) * v[3];
       if constexpr (sizeof(T) == 2) *reinterpret_cast<uint32_t*>(o) = f2bf2(a, b);
       else *reinterpret_cast<float2*>(o) = make_float2(a, b);
       break;
@@ -167,6 +176,84 @@ __device__ __forceinline__ void epilogue(const GemmArgs& g, int group, int m, in
       const f32x4 b = *reinterpret_cast<const f32x4*>(l.mid_b + n);
 #pragma unroll
       for (int i = 0; i < 4; ++i) v[i] = expf(-expf(v[i] + b[i]));
+      store4(g.f0 + static_cast<size_t>(m) * g.ldo + n, v);
+      break;
+    }
+    case EPI_CAPPED_LOGITS: {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) v[i] = soft_cap(v[i] * g.logit_scale, g.logit_softcap);
+      store4(g.f0 + static_cast<size_t>(m) * g.ldo + n, v);
+      break;
+    }
+    case EPI_ADD: {
+      float* x = g.f0 + static_cast<size_t>(m) * g.ldo + n;
+      store4(x, read4(x) + v);
+      break;
+    }
+    case EPI_ATTENTION_IN: {
+      const int q_rows = l.heads * l.q_stride, k_rows = l.kv_heads * l.head_dim, v_rows = l.kv_heads * l.v_dim, row = l.head_dim + l.v_dim, pos = g.position + m;
+      T* cache = static_cast<T*>(l.cache) + (static_cast<size_t>(g.slot) * l.ring + pos % l.ring) * l.kv_heads * row;
+      if (n < q_rows + k_rows) {
+        const int d = n < q_rows ? n % l.q_stride : (n - q_rows) % l.head_dim;
+        float e[4] = {v[0], v[1], v[2], v[3]};
+        rotate(l, pos, d, e[0], e[1]);
+        rotate(l, pos, d + 2, e[2], e[3]);
+        v = f32x4{e[0], e[1], e[2], e[3]};
+        store4(n < q_rows ? static_cast<T*>(g.out) + static_cast<size_t>(m) * q_rows + n : cache + (n - q_rows) / l.head_dim * row + d, v);
+      } else if (n < q_rows + k_rows + v_rows) {
+        const int c = n - q_rows - k_rows;
+        store4(cache + c / l.v_dim * row + l.head_dim + c % l.v_dim, v);
+      } else {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v[i] = sigmoid(v[i]);
+        store4(static_cast<T*>(g.out2) + static_cast<size_t>(m) * l.mix_width + n - q_rows - k_rows - v_rows, v);
+      }
+      break;
+    }
+    case EPI_DELTA_IN: {
+      const int channels = conv_channels(l), ranks = l.rank + l.gate_rank;
+      if (n < channels) {
+        store4(static_cast<T*>(g.out) + static_cast<size_t>(m) * channels + n, v);
+      } else if (n < channels + ranks) {
+        store4(static_cast<T*>(g.out2) + static_cast<size_t>(m) * ranks + n - channels, v);
+      } else {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v[i] = sigmoid(v[i]);
+        store4(g.f0 + static_cast<size_t>(m) * g.ldo + n - channels - ranks, v);
+      }
+      break;
+    }
+    case EPI_DELTA_MID: {
+      const int per = l.head_dim + l.v_dim, head = n / per, c = n % per;
+      if (c < l.head_dim) {
+        const f32x4 b = *reinterpret_cast<const f32x4*>(l.mid_b + head * l.head_dim + c);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v[i] = delta_decay(l, head, v[i] + b[i]);
+        store4(g.f0 + static_cast<size_t>(m) * l.heads * l.head_dim + head * l.head_dim + c, v);
+      } else {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v[i] = sigmoid(v[i]);
+        store4(static_cast<T*>(g.out) + static_cast<size_t>(m) * l.mix_width + head * l.v_dim + c - l.head_dim, v);
+      }
+      break;
+    }
+    case EPI_GLA_IN: {
+      const int qkv = 2 * l.heads * l.head_dim + l.mix_width;
+      if (n < qkv) {
+        store4(g.f0 + static_cast<size_t>(m) * qkv + n, v);
+      } else if (n < qkv + l.mix_width) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v[i] *= sigmoid(v[i]);
+        store4(static_cast<T*>(g.out) + static_cast<size_t>(m) * l.mix_width + n - qkv, v);
+      } else {
+        store4(static_cast<T*>(g.out2) + static_cast<size_t>(m) * l.rank + n - qkv - l.mix_width, v);
+      }
+      break;
+    }
+    case EPI_GLA_MID: {
+      const f32x4 b = *reinterpret_cast<const f32x4*>(l.mid_b + n);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) v[i] = gla_decay(l, v[i] + b[i]);
       store4(g.f0 + static_cast<size_t>(m) * g.ldo + n, v);
       break;
     }
@@ -515,18 +602,25 @@ __global__ __launch_bounds__(kPfThreads) void latent_rows(const float* raw, QmkH
   }
 }
 
+// Keys of an attention: key j of key head h at at[j * pitch + h * head]; heads_per query heads share a key head.
+template <class T>
+struct Keys {
+  const T* at;
+  int pitch, head, heads_per;
+};
+
 // Windowed attention over expanded keys: 64 queries of one head a workgroup (16 a wave), 32 keys a step.
 // Scores are computed transposed (keys x queries), so a lane holds eight weights of ONE query in exactly the shape the
 // value product's second operand wants, with keys in the order 4g..4g+3, 16+4g..16+4g+3.
 template <class T, int QT, int VT>   // most 32-column steps of a query, most 16-row tiles of a value
-__global__ __launch_bounds__(kPfThreads) void window_attention(const T* q, const T* k_nope, const T* rows, const T* v_t, const T* gate, QmkHybridLayer l,
+__global__ __launch_bounds__(kPfThreads) void window_attention(const T* q, Keys<T> keys, const T* rows, const T* v_t, const T* gate, QmkHybridLayer l,
                                                                int first, int position, int M, int keys_cap, T* out) {
   constexpr int kKeys = 32;
   constexpr int kPadK = 16 / sizeof(T), kPadV = 16 / sizeof(T);
   __shared__ __align__(16) T sk[kKeys][QT * 32 + kPadK];
   __shared__ __align__(16) T sv[VT * 16][kKeys + kPadV];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g = lane >> 4, col = lane & 15;
-  const int head = blockIdx.y, q0 = blockIdx.x * 64;
+  const int head = blockIdx.y, kv = head / keys.heads_per, q0 = blockIdx.x * 64;
   const int dq = l.q_stride, steps = dq / 32, vt = l.v_dim / 16, width = l.rank + l.rot_dim;
   const int m = q0 + wave * 16 + col, pos = position + m;
   Frag<T> fq[QT];
@@ -553,8 +647,8 @@ __global__ __launch_bounds__(kPfThreads) void window_attention(const T* q, const
     k_at[i] = nullptr;                 // columns behind the rotated part: zeros
     k_step[i] = 0;
     if (c < l.head_dim) {
-      k_at[i] = k_nope + static_cast<size_t>(row) * l.heads * l.head_dim + head * l.head_dim + c;
-      k_step[i] = kKeys * l.heads * l.head_dim;
+      k_at[i] = keys.at + static_cast<size_t>(row) * keys.pitch + kv * keys.head + c;
+      k_step[i] = kKeys * keys.pitch;
     } else if (c < l.head_dim + l.rot_dim) {
       k_at[i] = rows + static_cast<size_t>(row) * width + l.rank + c - l.head_dim;
       k_step[i] = kKeys * width;
@@ -572,7 +666,7 @@ __global__ __launch_bounds__(kPfThreads) void window_attention(const T* q, const
     for (int i = 0; i < kVLoads; ++i) {
       const int id = i * kPfThreads + tid, r = id / (kKeys / kU), c = id % (kKeys / kU) * kU;
       rv[i] = v4u{0u, 0u, 0u, 0u};
-      if (r < l.v_dim && base + c < hi) rv[i] = *reinterpret_cast<const v4u*>(v_t + static_cast<size_t>(head * l.v_dim + r) * keys_cap + base - first + c);
+      if (r < l.v_dim && base + c < hi) rv[i] = *reinterpret_cast<const v4u*>(v_t + static_cast<size_t>(kv * l.v_dim + r) * keys_cap + base - first + c);
       if (base + c + kU > hi) {   // keys behind the last one: whatever the buffer holds there must not enter a sum
         T* e = reinterpret_cast<T*>(&rv[i]);
 #pragma unroll

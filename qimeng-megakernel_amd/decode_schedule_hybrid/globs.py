@@ -1,7 +1,8 @@
 """``Globals`` of the hybrid route: weights, per-slot states, buffers and the layer table the kernels read.
 
 Unlike the routes of uniform layers, whose tensors are stacked over layers, every layer here has sizes of its own:
-``layer_weights[i]`` / ``layer_state[i]`` hold a layer's tensors by the field names of ``QmkHybridLayer``
+``layer_weights[i]`` / ``layer_state[i]`` hold the tensors of entry ``i`` of the shape (a layer, or a branch of one in one
+of its passes: passes share weights and have states of their own) by the field names of ``QmkHybridLayer``
 (``include/qmk_hybrid.h``), and ``build_globals`` writes their addresses into one table, kept on both sides.
 """
 from __future__ import annotations
@@ -48,9 +49,9 @@ class Globals:
 
 def state_tensors(shape: HybridShape, i: int, *, slots: int, max_positions: int, portion_rows: int, dtype: torch.dtype,
                   device: torch.device | str) -> dict[str, Tensor]:
-    """The per-slot state of layer ``i``.  The cache of a windowed attention is a ring: it holds the keys the window can
+    """The per-slot state of entry ``i``.  The cache of a windowed attention is a ring: it holds the keys the window can
     still reach while a whole portion's rows are written, and no more."""
-    l = shape.layers[i]
+    l = shape.entries[i].shape
 
     def zeros(*size: int, dtype: torch.dtype = torch.float32) -> Tensor:
         return torch.zeros(*size, dtype=dtype, device=device)
@@ -58,6 +59,14 @@ def state_tensors(shape: HybridShape, i: int, *, slots: int, max_positions: int,
     if l.type == "latent_attention":
         ring = min(max_positions, min(l.window, max_positions) - 1 + portion_rows)
         return {"cache": zeros(slots, ring, l.rank_s + l.rot_s, dtype=dtype)}
+    if l.type == "attention":
+        return {"cache": zeros(slots, max_positions, l.kv_heads, l.dim_s + l.v_s, dtype=dtype)}
+    if l.type == "gla":
+        return {"state": zeros(slots, l.heads, l.dim_s, l.v_s)}
+    if l.type == "delta":
+        return {"state": zeros(slots, l.heads, l.dim_s, l.v_s), "shift": zeros(slots, 2, l.taps - 1, l.conv_channels)}
+    if l.type in ("join", "final"):
+        return {}
     if l.type == "rglru":
         return {"state": zeros(slots, l.mix_width), "shift": zeros(slots, 2, max(l.taps - 1, 1), l.mix_width)[:, :, : l.taps - 1].contiguous()}
     return {"state": zeros(slots, l.heads, l.dim_s, l.dim_s), "shift": zeros(slots, 2, shape.width_s)}
@@ -72,13 +81,13 @@ def build_globals(shape: HybridShape, packed: dict[str, Any], *, dtype: torch.dt
     portion_rows = max(1, min(portion_rows, max_positions))
     g = Globals(shape=shape, dtype=dtype, slots=slots, max_positions=max_positions, portion_rows=portion_rows)
     g.embed_tokens, g.lm_head_weights, g.lm_head_norm_weights = packed["embed"], packed["head"], packed["final_norm"]
-    tables: dict[tuple[int, float], tuple[Tensor, Tensor]] = {}
-    for i, l in enumerate(shape.layers):
-        w = dict(packed["layers"][i])
-        if l.type == "latent_attention":
-            key = (l.rot_dim, l.rope_base)
+    tables: dict[tuple, tuple[Tensor, Tensor]] = {}
+    for i, e in enumerate(shape.entries):
+        l, w = e.shape, dict(packed["layers"][i])
+        if l.type in ("latent_attention", "attention"):
+            key = (l.rot_dim, l.rope_base, l.rope_scaling)
             if key not in tables:
-                cos, sin = rope_tables(l.rot_dim, l.rope_base, max_positions)
+                cos, sin = rope_tables(l.rot_dim, l.rope_base, max_positions, l.rope_scaling)
                 tables[key] = (cos.to(device), sin.to(device))
             w["rope_cos"], w["rope_sin"] = tables[key]
         g.layer_weights.append(w)

@@ -1,8 +1,9 @@
-"""The nine opcodes of the hybrid decode route and their stage protocol.
+"""The opcodes of the hybrid decode route and their stage protocol.
 
 Every instruction carries the same nine operands.  ``layer`` indexes the layer table; ``sub`` is the wkv input (r, k, v,
-g, decay), the gate block, the head, the group of sixteen heads, or 0 / 1 for the output / down projection; ``start`` and
-``count`` are output rows (pairs of rows for opcodes 2 and 8, part number and number of parts for opcode 4).
+g, decay), the gate block, the head, the group of at most sixteen heads (of one key head, where there are several), or
+0 / 1 for the output / down projection; ``start`` and ``count`` are output rows (pairs of rows for opcodes 2 and 8, part
+number and number of parts for opcode 4).
 
 A step is a chain of stages.  An instruction waits until ``wait_count`` arrivals are counted on ``wait_stage`` (-1: none)
 and counts one arrival on ``arrive_stage``; the schedule's stages are all-to-all, so ``wait_count`` is the number of
@@ -37,7 +38,7 @@ class StageInstruction(Instruction):
 @dataclass
 class RMS_InProject(StageInstruction):
     """Norm + the mixer's stacked input projections; convolution, rotation, gates where they act per output.
-    ``extra`` = 1: also keeps the normed input for the next token (wkv)."""
+    ``extra`` = 1: also keeps the normed input for the next token (wkv), or the residual for its next reader (plain)."""
     OPCODE: ClassVar[int] = 1
 
 
@@ -53,8 +54,8 @@ class LatentAbsorb(StageInstruction):
 
 
 @dataclass
-class LatentAttendSplitKV(StageInstruction):
-    """``extra``: which 128 columns of the latent."""
+class AttendSplitKV(StageInstruction):
+    """Over latents or over keys and values.  ``extra``: which 128 columns of the latent or value."""
     OPCODE: ClassVar[int] = 4
 
 
@@ -71,6 +72,7 @@ class WkvStep(StageInstruction):
 
 @dataclass
 class OutProject_Streams(StageInstruction):
+    """On a plain residual the rows are left for the residual's next reader to add."""
     OPCODE: ClassVar[int] = 7
 
 
@@ -84,5 +86,23 @@ class RMS_LMHead(StageInstruction):
     OPCODE: ClassVar[int] = 9
 
 
-INSTRUCTIONS = {c.OPCODE: c for c in (NoOp, RMS_InProject, GatedRecurrence, LatentAbsorb, LatentAttendSplitKV, LatentValue, WkvStep,
-                                      OutProject_Streams, RMS_UpGate_Gelu, RMS_LMHead)}
+@dataclass
+class GatedStateStep(StageInstruction):
+    """One head of a gated linear attention or gated delta rule: decay, recurrence, per-head norm and gate."""
+    OPCODE: ClassVar[int] = 10
+
+
+@dataclass
+class AttendMerge(StageInstruction):
+    """Merge of ``count`` parts of one head and the output gate."""
+    OPCODE: ClassVar[int] = 11
+
+
+@dataclass
+class JoinProject(StageInstruction):
+    """Rows of the residual a pass of the loop starts from."""
+    OPCODE: ClassVar[int] = 12
+
+
+INSTRUCTIONS = {c.OPCODE: c for c in (NoOp, RMS_InProject, GatedRecurrence, LatentAbsorb, AttendSplitKV, LatentValue, WkvStep,
+                                      OutProject_Streams, RMS_UpGate_Gelu, RMS_LMHead, GatedStateStep, AttendMerge, JoinProject)}

@@ -1,10 +1,14 @@
 """Instruction queues of one hybrid decode step.
 
-A layer is a chain of stages: input projections, the mixer's middle (recurrence; absorb, attend, value; wkv step), output
-projection, and for a feed-forward up/gate and down; the LM head ends the step.  Each stage's output rows are cut into
+A layer on residual streams is a chain of stages: input projections, the mixer's middle (recurrence; absorb, attend, value;
+wkv step), output projection, and for a feed-forward up/gate and down.  A layer run on the plain residual, whose branches and
+feed-forward read the same input, is three or four stages: all input projections and up/gate; state steps and attention;
+merges, the output projections of the state branches and down; the output projections of the attention.  (Without an
+attention the down projection runs beside the state steps, and the output projections follow.)  What a run leaves is added by
+the stage that reads the residual next.  The LM head ends the step.  Each stage's output rows are cut into
 blocks of equal size, about one per queue, and dealt to the queues from queue 0 on (the leaders of the per-XCD waits are
 the first eight queues, so they take part in every stage).  All output and down projections are cut alike: a queue owns its
-rows of the residual streams for the whole step, and the kernel relies on it.  One tensor serves every position: the split of the visible
+rows of the residual streams for the whole step, and the kernel relies on it (a plain residual has no such rows).  One tensor serves every position: the split of the visible
 keys over the parts of opcode 4 is worked out on the device.
 """
 from __future__ import annotations
@@ -50,12 +54,13 @@ class HybridScheduler:
     max_positions: int = 1 << 30
 
     def parts(self, layer: int) -> int:
-        """Parts the visible keys of a latent attention are cut into."""
-        reach = min(self.shape.layers[layer].window, self.max_positions)
+        """Parts the visible keys of an attention are cut into."""
+        l = self.shape.entries[layer].shape
+        reach = min(l.window, self.max_positions) if l.type == "latent_attention" else self.max_positions
         return max(1, min(MAX_PARTS, _ceil_div(reach, KEYS_PER_PART)))
 
     def max_parts(self) -> int:
-        return max([self.parts(i) for i, l in enumerate(self.shape.layers) if l.type == "latent_attention"], default=1)
+        return max([self.parts(i) for i, e in enumerate(self.shape.entries) if e.type in ("latent_attention", "attention")], default=1)
 
     def layer_stages(self, i: int) -> list[list[D.StageInstruction]]:
         l, q = self.shape.layers[i], self.queues
@@ -73,7 +78,7 @@ class HybridScheduler:
             stages.append([D.LatentAbsorb(i, h, a, n) for h, a, n in cut([(h, l.rank_s) for h in range(l.heads)], q)])
             stages[-1][0].extra = 1
             parts = self.parts(i)
-            stages.append([D.LatentAttendSplitKV(i, g, part, parts, extra=c) for g in range(_ceil_div(l.heads, 16)) for part in range(parts)
+            stages.append([D.AttendSplitKV(i, g, part, parts, extra=c) for g in range(_ceil_div(l.heads, 16)) for part in range(parts)
                            for c in range(_ceil_div(l.rank_s, ATTEND_COLUMNS))])
             stages.append([D.LatentValue(i, h, a, n, extra=parts) for h, a, n in cut([(h, l.v_s) for h in range(l.heads)], q)])
         D_s = self.shape.width_s
@@ -83,9 +88,55 @@ class HybridScheduler:
             stages.append([D.OutProject_Streams(i, 1, a, n) for _, a, n in cut([(0, D_s)], q, most=MAX_OUT_ROWS)])
         return stages
 
+    def _spread(self, parts: Sequence[tuple[int, Any]], busy: int = 0) -> list[D.StageInstruction]:
+        """Row instructions of one stage, cut alike: ``parts`` are (rows, instruction of a start and a count); ``busy`` other
+        instructions of the stage come before them."""
+        queues = max(self.queues - busy, self.queues // 2, 1)
+        return [parts[s][1](a, n) for s, a, n in cut([(k, rows) for k, (rows, _) in enumerate(parts)], queues)]
+
+    def run_stages(self, first: int) -> list[list[D.StageInstruction]]:
+        """Stages of the layer run whose branches start at entry ``first`` (plain residual)."""
+        head = self.shape.entries[first]
+        branches = {i: self.shape.entries[i].shape for i in range(first, first + head.branches)}
+        width, ff = self.shape.width_s, self.shape.layers[head.layer].ff_s if head.ff else 0
+        rows: list[tuple[int, Any]] = [(l.in_rows, lambda a, n, i=i: D.RMS_InProject(i, 0, a, n)) for i, l in branches.items()]
+        down: list[tuple[int, Any]] = []
+        if ff:
+            rows.append((2 * ff, lambda a, n: D.RMS_UpGate_Gelu(first, 0, a // 2, n // 2)))
+            down.append((width, lambda a, n: D.OutProject_Streams(first, 1, a, n)))
+        stages = [self._spread(rows)]
+        stages[0][0].extra = 1
+        steps: list[D.StageInstruction] = []
+        merges: list[D.StageInstruction] = []
+        early: list[tuple[int, Any]] = []
+        late: list[tuple[int, Any]] = []
+        for i, l in branches.items():
+            out = (width, lambda a, n, i=i: D.OutProject_Streams(i, 0, a, n))
+            if l.type == "attention":
+                parts, blocks = self.parts(i), _ceil_div(l.heads // l.kv_heads, 16)
+                steps += [D.AttendSplitKV(i, g, part, parts, extra=c) for part in range(parts) for g in range(l.kv_heads * blocks)
+                          for c in range(_ceil_div(l.v_s, ATTEND_COLUMNS))]
+                merges += [D.AttendMerge(i, h, 0, parts) for h in range(l.heads)]
+                late.append(out)
+            else:
+                steps = [D.GatedStateStep(i, h, 0, 1) for h in range(l.heads)] + steps
+                early.append(out)
+        if merges:
+            stages += [steps, merges + self._spread(early + down, len(merges)), self._spread(late)]
+        else:
+            stages += [steps + (self._spread(down, len(steps)) if down else []), self._spread(early)]
+        return stages
+
     def stages(self) -> list[list[D.StageInstruction]]:
-        out = [s for i in range(len(self.shape.layers)) for s in self.layer_stages(i)]
-        last = len(self.shape.layers) - 1
+        out: list[list[D.StageInstruction]] = []
+        last = len(self.shape.entries) - 1
+        if not self.shape.plain:
+            out = [s for i in range(len(self.shape.layers)) for s in self.layer_stages(i)]
+        for i, e in enumerate(self.shape.entries if self.shape.plain else ()):
+            if e.type == "join":
+                out.append(self._spread([(self.shape.width_s, lambda a, n: D.JoinProject(i, 0, a, n))]))
+            elif e.type != "final" and e.branch == 0:
+                out += self.run_stages(i)
         out.append([D.RMS_LMHead(last, 0, a, n) for _, a, n in cut([(0, self.shape.vocab_s)], self.queues)])
         for k, stage in enumerate(out):
             for ins in stage:

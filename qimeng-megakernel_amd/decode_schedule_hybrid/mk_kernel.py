@@ -18,6 +18,7 @@ from .instructions import scheduler as _scheduler
 
 _LIBRARY_NAME = "libqmk_hybrid.so"
 _P, _I, _F = ctypes.c_void_p, ctypes.c_int32, ctypes.c_float
+QMK_NORM_LAYER = QMK_ACT_SILU = 1      # include/qmk_hybrid.h
 _ERRORS = {1: "null argument", 2: "struct_size does not match the library", 3: "dimension out of range", 4: "position outside the request's capacity",
            5: "more instruction queues than co-resident workgroups", 6: "no usable HIP device", 7: "kernel launch failed", 8: "unknown element type",
            9: "workspace too small", 32: "device: unknown opcode", 33: "device: instruction operand out of bounds",
@@ -25,7 +26,7 @@ _ERRORS = {1: "null argument", 2: "struct_size does not match the library", 3: "
 
 #: pointer fields of the layer table = keys of a layer's weight and state tensors
 _LAYER_POINTERS = ("norm1", "norm2", "in_w", "in_b", "mid_w", "mid_b", "uk_w", "uv_w", "o_w", "mlp_w", "down_w", "vec0", "vec1", "vec2", "rope_cos",
-                   "rope_sin", "hc", "next1", "next2", "cache", "state", "shift")
+                   "rope_sin", "hc", "next1", "next2", "out_norm", "cache", "state", "shift")
 
 
 class QmkHybridLayer(ctypes.Structure):
@@ -33,7 +34,9 @@ class QmkHybridLayer(ctypes.Structure):
 
     _fields_ = [(n, _I) for n in ("type", "has_mlp", "in_rows", "mix_width", "heads", "head_dim", "head_dim_true", "rot_dim", "rot_true", "q_stride",
                                   "v_dim", "rank", "rank_true", "window", "ring", "taps", "blocks", "block_dim", "ff")]
-    _fields_ += [("scale", _F)] + [(n, _P) for n in _LAYER_POINTERS]
+    _fields_ += [("scale", _F)]
+    _fields_ += [(n, _I) for n in ("kv_heads", "v_true", "gate_rank", "norm", "act", "branch", "branches", "prev", "x_from", "x_to", "proj_at", "mix_at", "ff_at")]
+    _fields_ += [(n, _F) for n in ("q_scale", "decay_scale", "out_scale")] + [(n, _P) for n in _LAYER_POINTERS]
 
 
 class QmkHybridArgs(ctypes.Structure):
@@ -43,7 +46,7 @@ class QmkHybridArgs(ctypes.Structure):
     _fields_ += [("layers", _P), ("layers_device", _P)]
     _fields_ += [(n, _I) for n in ("num_layers", "width", "width_true", "streams", "vocab", "vocab_rows", "slots", "slot", "position", "max_positions",
                                    "flip", "tokens", "num_want", "portion_rows")]
-    _fields_ += [("eps", _F), ("reserved0", _I)]
+    _fields_ += [("eps", _F), ("logit_scale", _F), ("logit_softcap", _F), ("reserved0", _I)]
     _fields_ += [(n, _P) for n in ("embed", "final_norm", "head", "token_in", "token_out", "want", "logits", "layer_out", "workspace")]
     _fields_ += [("workspace_bytes", ctypes.c_uint64), ("instructions", _P), ("barriers", _P)]
     _fields_ += [(n, _I) for n in ("num_queues", "num_insts", "barrier_groups", "max_splits")]
@@ -71,19 +74,38 @@ def load_library(mk_dir: Path | None = None) -> ctypes.CDLL:
 
 
 def layer_table(globs: Globals) -> ctypes.Array:
-    """The layer table of ``globs``: sizes from the shape, pointers from the tensors."""
-    table = (QmkHybridLayer * len(globs.shape.layers))()
-    for i, l in enumerate(globs.shape.layers):
-        e = table[i]
-        e.type, e.has_mlp, e.in_rows, e.mix_width, e.ff = l.mixer, int(l.ff > 0), l.in_rows, l.mix_width, l.ff_s
-        e.heads = l.heads
+    """The layer table of ``globs``, one entry per entry of its shape: sizes from the shape, pointers from the tensors."""
+    entries = globs.shape.entries
+    table = (QmkHybridLayer * len(entries))()
+    proj_at = mix_at = 0
+    for i, entry in enumerate(entries):
+        e, l = table[i], entry.shape
+        e.type, e.has_mlp, e.ff = l.mixer, int(entry.ff > 0), globs.shape.layers[entry.layer].ff_s if entry.ff else 0
+        if globs.shape.plain:   # a run's branches side by side in the buffers of a step, its feed-forward behind them
+            if entry.branch == 0:
+                proj_at = mix_at = 0
+            e.norm, e.act = QMK_NORM_LAYER, QMK_ACT_SILU
+            e.branch, e.branches, e.prev, e.x_from, e.x_to = entry.branch, entry.branches, entry.prev, entry.x_from, entry.x_to
+            e.out_scale = 1.0 / entry.branches
+            e.proj_at, e.mix_at = proj_at, mix_at
+        if l.type not in ("join", "final"):
+            e.in_rows, e.mix_width, e.heads, e.kv_heads = l.in_rows, l.mix_width, l.heads, l.kv_heads
+            proj_at, mix_at = proj_at + l.in_rows, mix_at + l.mix_width
+        if entry.ff and globs.shape.plain:
+            e.ff_at = sum(b.shape.mix_width for b in entries[i : i + entry.branches])
         if l.type == "latent_attention":
             e.head_dim, e.rot_dim, e.rot_true, e.q_stride, e.v_dim = l.dim_s, l.rot_s, l.rot_dim, l.q_stride, l.v_s
             e.rank, e.rank_true, e.scale = l.rank_s, l.rank, l.scale
             e.window, e.ring = min(l.window, globs.max_positions), globs.layer_state[i]["cache"].shape[1]
+        elif l.type == "attention":
+            e.head_dim, e.rot_true, e.q_stride, e.v_dim, e.scale = l.dim_s, l.rot_dim, l.q_stride, l.v_s, l.scale
+            e.window, e.ring = globs.max_positions, globs.layer_state[i]["cache"].shape[1]
+        elif l.type in ("delta", "gla"):
+            e.head_dim, e.v_dim, e.v_true, e.rank, e.gate_rank, e.taps = l.dim_s, l.v_s, l.v_dim, l.rank_s, l.gate_rank_s, l.taps
+            e.q_scale, e.decay_scale = l.dim**-0.5, 1.0 / l.tau if l.tau else 0.0
         elif l.type == "rglru":
             e.taps, e.blocks, e.block_dim = l.taps, l.blocks, l.block_s
-        else:
+        elif l.type == "wkv":
             e.head_dim, e.head_dim_true, e.rank = l.dim_s, l.dim, l.rank_s
         tensors = {**globs.layer_weights[i], **globs.layer_state[i]}
         for name, t in tensors.items():
@@ -126,8 +148,8 @@ class HybridMegaKernel:
         a.struct_size = ctypes.sizeof(QmkHybridArgs)
         a.dtype = 1 if g.dtype == torch.float32 else 0
         a.layers, a.layers_device = ctypes.addressof(self._table), self._table_device.data_ptr()
-        a.num_layers, a.width, a.width_true, a.streams = len(s.layers), s.width_s, s.width, s.streams
-        a.vocab, a.vocab_rows, a.eps = s.vocab, s.vocab_s, s.eps
+        a.num_layers, a.width, a.width_true, a.streams = len(s.entries), s.width_s, s.width, s.streams
+        a.vocab, a.vocab_rows, a.eps, a.logit_scale, a.logit_softcap = s.vocab, s.vocab_s, s.eps, s.logit_scale, s.logit_softcap
         a.slots, a.max_positions, a.portion_rows = g.slots, g.max_positions, g.portion_rows
         a.embed, a.final_norm, a.head = g.embed_tokens.data_ptr(), g.lm_head_norm_weights.data_ptr(), g.lm_head_weights.data_ptr()
         a.instructions, a.barriers = g.instructions.data_ptr(), g.barriers.data_ptr()
@@ -181,8 +203,8 @@ class HybridMegaKernel:
         M = int(tokens.numel())
         if not 1 <= M <= g.portion_rows:
             raise ValueError(f"a portion holds 1..{g.portion_rows} tokens, got {M}")
-        if layer_out is not None and tuple(layer_out.shape) != (len(g.shape.layers), M, g.shape.width_s):
-            raise ValueError("layer_out must be [layers, tokens, storage width]")
+        if layer_out is not None and tuple(layer_out.shape) != (g.shape.run_count, M, g.shape.width_s):
+            raise ValueError("layer_out must be [layer runs, tokens, storage width]")
         logits = torch.empty(n, g.shape.vocab_s, dtype=torch.float32, device=g.device)
         a = self._args
         a.slot, a.position, a.flip, a.tokens, a.num_want = g.slot, g.position_id, g.flip, M, n

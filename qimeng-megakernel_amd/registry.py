@@ -38,10 +38,12 @@ MODELS: dict[str, tuple[Family, str, str]] = {
     "qwen3-30b-a3b": (MOE, "decode_schedule_moe.model_config", "QWEN3_30B_A3B"),
     "lusupel-1b": (HYBRID, "synthetic", "LUSUPEL_1B"),
     "lusupel-2b": (HYBRID, "synthetic", "LUSUPEL_2B"),
+    "givopel-1b": (HYBRID, "synthetic", "GIVOPEL_1B"),
+    "givopel-2b": (HYBRID, "synthetic", "GIVOPEL_2B"),
 }
 
 #: ``architecture`` of a model folder's config.json -> family
-ARCHITECTURES: dict[str, Family] = {"Lusupel": HYBRID}
+ARCHITECTURES: dict[str, Family] = {"Lusupel": HYBRID, "Givopel": HYBRID}
 
 
 def shape_of(name: str) -> Any:

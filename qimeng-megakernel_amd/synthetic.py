@@ -314,10 +314,38 @@ def hybrid_shape(pattern: str, *, width: int, vocab: int, streams: int, eps: flo
     return HybridShape(layers=tuple(LayerShape(ff=ff.get(c, 0), **kinds[c]) for c in pattern), width=width, vocab=vocab, streams=streams, eps=eps)
 
 
+def looped_shape(pattern: str, *, width: int, vocab: int, eps: float = 1e-6, ff: dict[str, int] | None = None, loop: tuple[int, int, int] | None = None,
+                 logit_scale: float = 1.0, logit_softcap: float = 0.0, heads: int = 16, kv_heads: int = 8, dim: int = 128, v_dim: int = 128,
+                 rot_dim: int | None = None, rope_base: float = 10000.0, rope_scaling: tuple[float, float, float, float] | None = None,
+                 scale: float | None = None, delta_heads: int = 16, delta_kv_heads: int = 16, delta_dim: int = 128, delta_v_dim: int = 128, taps: int = 4,
+                 delta_rank: int = 128, gate_rank: int = 128, gla_heads: int = 8, gla_dim: int = 128, gla_v_dim: int = 256, gla_rank: int = 16,
+                 tau: float = 16.0) -> HybridShape:
+    """A looped hybrid shape from a string of layers: ``p`` softmax attention beside a gated delta rule, ``g`` gated linear
+    attention; ``ff`` gives the feed-forward size per letter (absent: none)."""
+    ff = ff or {}
+    attention = LayerShape("attention", heads=heads, kv_heads=kv_heads, dim=dim, v_dim=v_dim, rot_dim=dim if rot_dim is None else rot_dim, rope_base=rope_base,
+                           rope_scaling=rope_scaling, scale=dim ** -0.5 if scale is None else scale)
+    delta = LayerShape("delta", heads=delta_heads, kv_heads=delta_kv_heads, dim=delta_dim, v_dim=delta_v_dim, taps=taps, rank=delta_rank, gate_rank=gate_rank)
+    kinds = {
+        "p": dict(type="parallel", branches=(attention, delta)),
+        "g": dict(type="gla", heads=gla_heads, kv_heads=gla_heads, dim=gla_dim, v_dim=gla_v_dim, rank=gla_rank, tau=tau),
+    }
+    return HybridShape(layers=tuple(LayerShape(ff=ff.get(c, 0), **kinds[c]) for c in pattern), width=width, vocab=vocab, streams=0, eps=eps, loop=loop,
+                       logit_scale=logit_scale, logit_softcap=logit_softcap)
+
+
 #: about the parameters of the Llama-3.2-1B shape (width, feed-forward and vocabulary are its own)
 LUSUPEL_1B = hybrid_shape("raaw" * 4, width=2048, vocab=128256, streams=4, ff={"a": 8192, "r": 8192})
 #: about the parameters of the Qwen3-1.7B shape
 LUSUPEL_2B = hybrid_shape("raaw" * 7, width=2048, vocab=151936, streams=4, ff={"a": 6144, "r": 6144, "w": 6144}, window=2048)
+
+
+#: about the bytes per token of the Llama-3.2-1B shape (eleven layer runs, the loop's layers streamed once per pass)
+GIVOPEL_1B = looped_shape("ppgpgppg", width=2048, vocab=128256, ff={"p": 8192, "g": 8192}, loop=(2, 5, 2), rope_base=500000.0,
+                          rope_scaling=(8.0, 8192.0, 32.0, 1.0), logit_softcap=30.0)
+#: ... of the Qwen3-1.7B shape
+GIVOPEL_2B = looped_shape("ppgpgppgppgppg", width=2048, vocab=151936, ff={"p": 6144, "g": 6144}, loop=(4, 10, 2), rope_base=1000000.0,
+                          rope_scaling=(4.0, 8192.0, 32.0, 1.0), logit_softcap=30.0)
 
 
 def random_hybrid_weights(shape: HybridShape, seed: int, device: torch.device | str = "cpu") -> dict[str, torch.Tensor]:
@@ -359,9 +387,17 @@ def random_hybrid_weights(shape: HybridShape, seed: int, device: torch.device | 
             t = uniform(size, -6.0, 0.0)
         elif part == "mix.u":
             t = normal(size, 0.5)
-        elif part == "mix.conv":
+        elif part.endswith(".out"):             # a branch's norm (plain residual)
+            t = normal(size, 0.1, 1.0)
+        elif part.endswith("A_log"):
+            t = uniform(size, -2.0, 1.0)
+        elif part.endswith("dt_bias"):
+            t = uniform(size, -5.0, 0.0)
+        elif part == "mix.a2.b":
+            t = normal(size, 1.5, 1.0)
+        elif part.endswith("conv"):
             t = normal(size, size[-1] ** -0.5)
-        elif part.endswith(".b"):
+        elif part.endswith(".b") and not part.endswith("right.b"):     # (there it is a projection)
             t = normal(size, 0.1)
         else:
             t = normal(size, size[-1] ** -0.5)
