@@ -500,23 +500,79 @@ def moe_decode_rows(args, shape, name: str, globs, kv_capacity: int, new_tokens:
     }
 
 
-HYBRID_PEER = {"lusupel-1b": "llama-3.2-1b", "lusupel-2b": "qwen3-1.7b"}   # the closest dense model at equal size
+HYBRID_PEER = {"lusupel-1b": "llama-3.2-1b", "lusupel-2b": "qwen3-1.7b",   # the closest model at equal size
+               "givopel-1b": "lusupel-1b", "givopel-2b": "lusupel-2b"}
 
 
-def hybrid_decode(args) -> dict:
-    """Greedy decode and prefill of a hybrid (Lusupel) shape, beside the closest dense shape of about its size on the
-    same GPU: that one's decode through its own kernel, and its prefill, which is its decode kernel once per position."""
+def hybrid_prefill(globs, mk, lengths, gen) -> dict:
+    """Prefill throughput of random prompts, the best of three runs each."""
+    import torch
+
+    from qimeng_megakernel_amd import decode_hybrid
+    from qimeng_megakernel_amd.decode_schedule_hybrid.state import RequestTable
+
+    shape, table, out = globs.shape, RequestTable(globs), {}
+    for n in lengths:
+        ids = torch.randint(0, shape.vocab, (n,), generator=gen, dtype=torch.long).to(globs.device)
+        best = float("inf")
+        for it in range(4):
+            request = table.open("prefill")
+            a, b = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
+            a.record()
+            decode_hybrid.run_tokens(globs, mk, request, ids, [n - 1])
+            b.record()
+            torch.cuda.synchronize(globs.device)
+            table.close("prefill")
+            if it:
+                best = min(best, a.elapsed_time(b) / 1e3)
+        flops = shape.prefill_flops(n)
+        out[str(n)] = {"tok_s": n / best, "ms": best * 1e3, "tflops": flops / best / 1e12, "mfma_frac": flops / best / MFMA_PEAK_FLOPS}
+    return out
+
+
+def hybrid_peer(args, prompt, new_tokens: int, timed: int, lengths, gen) -> dict:
+    """Decode and prefill of the closest model: a dense shape through its own kernel (prefill is its decode kernel once per
+    position), or the hybrid route's other design."""
     import torch
 
     from qimeng_megakernel_amd import decode, decode_hybrid, registry, synthetic
-    from qimeng_megakernel_amd.decode_schedule import mk_kernel as dense_kernel
-    from qimeng_megakernel_amd.decode_schedule.model_config import LlamaConfig
+
+    device = torch.device("cuda:0")
+    name = HYBRID_PEER[args.model]
+    shape = registry.shape_of(name)
+    if name in HYBRID_PEER:
+        from qimeng_megakernel_amd.decode_schedule_hybrid import mk_kernel
+
+        globs = synthetic.build_synthetic_hybrid_globals(shape, seed=args.seed, max_positions=max([args.prompt_len + new_tokens] + lengths), portion_rows=4096,
+                                                         device=device)
+        mk = mk_kernel.get_mk()
+        decode_hybrid.decode(globs, prompt % shape.vocab, 17, mk=mk, decode_time=False)
+        t = decode_hybrid.decode(globs, prompt % shape.vocab, new_tokens, mk=mk, timed_steps=timed)["timing"]
+        prefill: dict = {"prefill": hybrid_prefill(globs, mk, lengths, gen)}
+    else:
+        from qimeng_megakernel_amd.decode_schedule import mk_kernel
+        from qimeng_megakernel_amd.decode_schedule.model_config import LlamaConfig
+
+        LlamaConfig.set_shape(shape)
+        globs = synthetic.build_globals(synthetic.random_weights(shape, args.seed, args.prompt_len + new_tokens), shape, args.prompt_len + new_tokens, device)
+        mk = mk_kernel.get_mk()
+        decode.decode(globs, prompt % shape.vocab_size, 17, mk=mk, decode_time=False)
+        t = decode.decode(globs, prompt % shape.vocab_size, new_tokens, mk=mk, device_sampling=True, timed_steps=timed)["timing"]
+        prefill = {"prefill_tok_s": t["kernel_tok_s"], "prefill": "its decode kernel once per prompt position"}
+    return {"model": name, "weight_bytes": shape.weight_bytes_per_token(), "kernel_tok_s": t["kernel_tok_s"], "ms_per_step": t["kernel_ms_per_step"],
+            "roofline_frac": t["achieved_GBps"] / HBM_PEAK_GBPS, **prefill}
+
+
+def hybrid_decode(args) -> dict:
+    """Greedy decode and prefill of a hybrid shape, beside the closest model of about its size on the same GPU."""
+    import torch
+
+    from qimeng_megakernel_amd import decode_hybrid, registry, synthetic
     from qimeng_megakernel_amd.decode_schedule_hybrid import mk_kernel
-    from qimeng_megakernel_amd.decode_schedule_hybrid.state import RequestTable
 
     device = torch.device("cuda:0")
     torch.cuda.set_device(device)
-    shape, peer_name = registry.shape_of(args.model), HYBRID_PEER[args.model]
+    shape = registry.shape_of(args.model)
     lengths = [int(x) for x in args.prefill_lengths.split(",") if x.strip()]
     new_tokens = max(args.new_tokens, args.steps + 1)
     timed = min(args.steps, new_tokens - 1)
@@ -537,48 +593,25 @@ def hybrid_decode(args) -> dict:
         if g_out["new_tokens"].tolist() != tokens:
             raise SystemExit("bench.py: the graph replay produced different tokens than the launch loop")
         graph_tok_s = g_out["timing"]["effective_tok_s_gpu"]
-
-    table, prefill = RequestTable(globs), {}
-    for n in lengths:
-        ids = torch.randint(0, shape.vocab, (n,), generator=gen, dtype=torch.long).to(device)
-        best = float("inf")
-        for it in range(4):
-            request = table.open("prefill")
-            a, b = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
-            a.record()
-            decode_hybrid.run_tokens(globs, mk, request, ids, [n - 1])
-            b.record()
-            torch.cuda.synchronize(device)
-            table.close("prefill")
-            if it:
-                best = min(best, a.elapsed_time(b) / 1e3)
-        flops = shape.prefill_flops(n)
-        prefill[str(n)] = {"tok_s": n / best, "ms": best * 1e3, "tflops": flops / best / 1e12, "mfma_frac": flops / best / MFMA_PEAK_FLOPS}
-    del globs
+    prefill = hybrid_prefill(globs, mk, lengths, gen)
+    del globs, out
     torch.cuda.empty_cache()
-
-    peer = registry.shape_of(peer_name)
-    LlamaConfig.set_shape(peer)
-    peer_globs = synthetic.build_globals(synthetic.random_weights(peer, args.seed, args.prompt_len + new_tokens), peer, args.prompt_len + new_tokens, device)
-    peer_mk = dense_kernel.get_mk()
-    decode.decode(peer_globs, prompt % peer.vocab_size, 17, mk=peer_mk, decode_time=False)
-    p = decode.decode(peer_globs, prompt % peer.vocab_size, new_tokens, mk=peer_mk, device_sampling=True, timed_steps=timed)["timing"]
+    peer = hybrid_peer(args, prompt, new_tokens, timed, lengths, gen)
     return {
         "metric": "kernel_tok_s", "value": t["kernel_tok_s"], "unit": "tok/s", "n_gpus": 1, "steps": timed, "warmup": args.warmup,
         "ms_per_step": t["kernel_ms_per_step"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
         "config": {"workload": f"{args.model} shape, batch-1 greedy decode, {args.prompt_len}-token prompt, {new_tokens} new tokens; timed: the last {timed} "
                                f"decode steps (contexts {t['first_timed_context']}..{t['last_timed_context']}), seeded random-init bf16 weights; prefill of "
                                f"random prompts in portions of up to 4096 tokens",
-                   "layers": len(shape.layers), "mixers": "".join({"rglru": "r", "latent_attention": "a", "wkv": "w"}[l.type] for l in shape.layers),
-                   "hidden": shape.width, "streams": shape.streams, "vocab": shape.vocab, "weight_bytes": shape.weight_bytes_per_token(), "batch": 1,
+                   "layers": len(shape.layers), "layer_runs": shape.run_count,
+                   "mixers": "".join({"rglru": "r", "latent_attention": "a", "wkv": "w", "parallel": "p", "gla": "g"}[l.type] for l in shape.layers),
+                   "hidden": shape.width, "streams": max(shape.streams, 1), "vocab": shape.vocab, "weight_bytes": shape.weight_bytes_per_token(), "batch": 1,
                    "seed": args.seed},
         "tok_s": t["effective_tok_s_wall"], "tok_s_gpu": t["effective_tok_s_gpu"], "kernel_tok_s": t["kernel_tok_s"], "tok_s_gpu_graph": graph_tok_s,
         "roofline": {"bound": "hbm", "achieved": t["achieved_GBps"], "peak": HBM_PEAK_GBPS, "unit": "GB/s", "frac": t["achieved_GBps"] / HBM_PEAK_GBPS,
                      "bytes_per_launch_avg": t["algorithmic_bytes"] / max(timed, 1), "kernel": "decode_megakernel_hybrid"},
         "prefill": prefill,
-        "closest_model": {"model": peer_name, "weight_bytes": peer.weight_bytes_per_token(), "kernel_tok_s": p["kernel_tok_s"],
-                          "ms_per_step": p["kernel_ms_per_step"], "roofline_frac": p["achieved_GBps"] / HBM_PEAK_GBPS,
-                          "prefill_tok_s": p["kernel_tok_s"], "prefill": "its decode kernel once per prompt position"},
+        "closest_model": peer,
     }
 
 
@@ -614,7 +647,7 @@ def hybrid_phase_table(name: str, context: int = 1000) -> dict:
             last = max(last, int(t[q, index[q], 2]))
             index[q] += 1
         ins = stage[0]
-        layer = shape.layers[ins.layer]
+        layer = shape.entries[ins.layer].shape
         kinds.append(type(ins).__name__ + {0: "", 1: "_down"}.get(ins.sub if ins.opcode() == 7 else 0, "") + ("" if ins.opcode() == 9 else ":" + layer.type))
         ends.append(last)
     start = int(t[..., 0][t[..., 0] > 0].min())
@@ -673,7 +706,7 @@ def main() -> None:
                          "(28 layers, per-head QK RMSNorm, tied LM head), the Qwen1.5-MoE-A2.7B shape with the MoE op set "
                          "(24 layers, 60 experts of 1408 with top-4 routing, shared expert of 5632), or the Qwen3-30B-A3B shape "
                          "(48 layers, 128 experts of 768 with renormalised top-8 routing, 32/4 heads of 128; 512 new tokens), "
-                         "or a hybrid (Lusupel) shape: decode and prefill, beside the dense shape of about its size")
+                         "or a hybrid (Lusupel, Givopel) shape: decode and prefill, beside the closest model of about its size")
     ap.add_argument("--prefill-lengths", default="512,2048,4096", help="hybrid shapes: prompt lengths whose prefill is timed")
     ap.add_argument("--host-sampling", action="store_true",
                     help="argmax and embedding lookup on the host between launches, as the reference's loop does "

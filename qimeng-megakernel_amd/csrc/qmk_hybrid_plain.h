@@ -291,7 +291,9 @@ __global__ __launch_bounds__(kPfThreads) void keep_inputs(const T* x, QmkHybridL
 }
 
 // One head and sixteen value columns a workgroup; a wave holds TILES tiles of sixteen key channels of the state as the
-// accumulators of the matrix instruction, which are also the second operand of the products that read it.
+// accumulators of the matrix instruction, which are also the second operand of the products that read it.  A wave's tiles
+// behind the last one are zeros and take part: with a branch around each tile's products this compiler has left out the wait
+// between a tile's last product and the first use of its result on the path that skips the next tile.
 template <int TILES, bool DELTA>
 __global__ __launch_bounds__(kChunkWaves * 64) void chunk_scan(const ChunkArgs g) {
   __shared__ f32x4 px[2][kChunkWaves][64], po[2][kChunkWaves][64];
@@ -345,13 +347,11 @@ __global__ __launch_bounds__(kChunkWaves * 64) void chunk_scan(const ChunkArgs g
     f32x4 x = {}, o = {};
     if constexpr (DELTA) {
 #pragma unroll
-      for (int j = 0; j < TILES; ++j)
-        if (j < mine) x = product(f.k[j], s[j], x);
+      for (int j = 0; j < TILES; ++j) x = product(f.k[j], s[j], x);
       px[buf][wave][lane] = x;
     }
 #pragma unroll
-    for (int j = 0; j < TILES; ++j)
-      if (j < mine) o = product(f.q[j], s[j], o);
+    for (int j = 0; j < TILES; ++j) o = product(f.q[j], s[j], o);
     po[buf][wave][lane] = o;
     __syncthreads();
     f32x4 u = f.v;
@@ -361,8 +361,7 @@ __global__ __launch_bounds__(kChunkWaves * 64) void chunk_scan(const ChunkArgs g
       u = product(f.t, u, f32x4{0.f, 0.f, 0.f, 0.f});
     }
 #pragma unroll
-    for (int j = 0; j < TILES; ++j)
-      if (j < mine) s[j] = product(f.d[j], u, s[j] * f.g[j]);
+    for (int j = 0; j < TILES; ++j) s[j] = product(f.d[j], u, s[j] * f.g[j]);
     if (wave == (chunk & (kChunkWaves - 1))) {
       o = product(f.b, u, f32x4{0.f, 0.f, 0.f, 0.f});
 #pragma unroll

@@ -240,8 +240,9 @@ def test_the_same_key_over_and_over():
     mk, g = mk_kernel.get_mk(), on_gpu(shape, w, torch.float32)
     tokens = [3] * 70 + [5, 3] * 20
     want = O.forward(shape.to_config(), w, torch.tensor(tokens), dtype=torch.float64)
+    rounding = error(O.forward(shape.to_config(), w, torch.tensor(tokens), dtype=torch.float32).double(), want)     # above the usual here
     for cuts in ([64, 46], [1] * 110):
-        assert error(run(g, mk, tokens, cuts), want) < TOL[torch.float32]
+        assert error(run(g, mk, tokens, cuts), want) < max(TOL[torch.float32], 4 * rounding)
 
 
 @BOTH
