@@ -648,6 +648,10 @@ def hybrid_phase_table(name: str, context: int = 1000) -> dict:
             index[q] += 1
         ins = stage[0]
         layer = shape.entries[ins.layer].shape
+        if shape.plain:     # a stage holds instructions of several kinds
+            kinds.append("+".join(dict.fromkeys(type(i).__name__ for i in stage)) + f" ({len(stage)})")
+            ends.append(last)
+            continue
         kinds.append(type(ins).__name__ + {0: "", 1: "_down"}.get(ins.sub if ins.opcode() == 7 else 0, "") + ("" if ins.opcode() == 9 else ":" + layer.type))
         ends.append(last)
     start = int(t[..., 0][t[..., 0] > 0].min())
@@ -701,7 +705,7 @@ def main() -> None:
     ap.add_argument("--length-bench-iters", type=int, default=5)
     ap.add_argument("--cpu-steps", type=int, default=16)
     ap.add_argument("--no-cpu-baseline", action="store_true")
-    ap.add_argument("--model", choices=("llama-3.2-1b", "qwen3-1.7b", "qwen1.5-moe-a2.7b", "qwen3-30b-a3b", "lusupel-1b", "lusupel-2b"), default="llama-3.2-1b",
+    ap.add_argument("--model", choices=("llama-3.2-1b", "qwen3-1.7b", "qwen1.5-moe-a2.7b", "qwen3-30b-a3b", "lusupel-1b", "lusupel-2b", "givopel-1b", "givopel-2b"), default="llama-3.2-1b",
                     help="layer geometry: the headline Llama-3.2-1B shape, the Qwen3-1.7B shape with the Qwen3 op set "
                          "(28 layers, per-head QK RMSNorm, tied LM head), the Qwen1.5-MoE-A2.7B shape with the MoE op set "
                          "(24 layers, 60 experts of 1408 with top-4 routing, shared expert of 5632), or the Qwen3-30B-A3B shape "

@@ -76,8 +76,8 @@ typedef struct QmkHybridLayer {
   int32_t prev;          /* plain residual: first entry of the run whose outputs are added to x before it is read, -1: none */
   int32_t x_from;        /* decode: the copy of x that is read (-1: the embedding) and the one that is left */
   int32_t x_to;
-  int32_t proj_at;       /* decode: first element of this entry's projections, of what its output projection reads and of */
-  int32_t mix_at;        /* its feed-forward's activations in the buffers of one step */
+  int32_t proj_at;       /* decode: first element of this entry's projections (delta: in_rows, then the output gate */
+  int32_t mix_at;        /* [heads * v_dim]), of what its mixer leaves and of its feed-forward's activations in a step's buffers */
   int32_t ff_at;
   float q_scale;         /* delta, gla: on the query */
   float decay_scale;     /* gla: on the logarithm of the decay */
@@ -90,9 +90,9 @@ typedef struct QmkHybridLayer {
                             gla: q, k [heads][head_dim], v, gate [heads][v_dim], decay rank; join: [D][2 D] */
   const float* in_b;     /* rglru: [in_rows], else NULL */
   const uint16_t* mid_w; /* rglru: [blocks][2 block_dim][block_dim], rows (ra_j, ri_j) interleaved;
-                            latent: W_uk per head transposed [heads * rank][head_dim]; wkv, gla: [heads * head_dim][rank];
-                            delta: [heads][head_dim | v_dim][rank | gate_rank], zeros off the diagonal blocks */
+                            latent: W_uk per head transposed [heads * rank][head_dim]; wkv, gla, delta: [heads * head_dim][rank] */
   const float* mid_b;    /* rglru: [blocks * 2 * block_dim] interleaved; wkv, delta, gla: the decay's constant [heads * head_dim] */
+  const uint16_t* gate_w;/* delta: [heads * v_dim][gate_rank] */
   const uint16_t* uk_w;  /* latent: [heads * head_dim][rank] */
   const uint16_t* uv_w;  /* latent: [heads * v_dim][rank] */
   const uint16_t* o_w;   /* [D][mix_width] */

@@ -31,7 +31,7 @@ __device__ __forceinline__ const DecodeParams& params_of_this_instruction() {
   return *(const DecodeParams*)args;   // the only kernel argument: offset 0 of the segment
 }
 
-template <class T>
+template <class T, bool PLAIN>
 __global__ __launch_bounds__(kThreads, 1) void decode_megakernel_hybrid(const DecodeParams p_launch) {
   const DecodeParams& p_loop = p_launch;
   __shared__ __align__(16) Smem s;
@@ -73,9 +73,13 @@ __global__ __launch_bounds__(kThreads, 1) void decode_megakernel_hybrid(const De
         case OP_UP_GATE:
         case OP_LM_HEAD:
         case OP_STATE_STEP:
-        case OP_JOIN: ok = op_rows<T>(p, s, o); break;
-        case OP_ATTEND: ok = op_attend<T>(p, s, o); break;
-        case OP_ATTEND_MERGE: ok = op_attend_merge(p, s, o); break;
+        case OP_JOIN:
+        case OP_GATE: ok = op_rows<T, PLAIN>(p, s, o); break;
+        case OP_ATTEND: ok = op_attend<T, PLAIN>(p, s, o); break;
+        case OP_ATTEND_MERGE:
+          if constexpr (PLAIN) ok = op_attend_merge(p, s, o);
+          else ok = bad_operand(p, o, o.opcode);
+          break;
         default:
           if (threadIdx.x == 0) report_error(counters_of(p), QMK_DEV_BAD_OPCODE, i, o.opcode, 0);
           ok = false;
@@ -143,14 +147,18 @@ int device_info(DeviceInfo** out) {
   DeviceInfo& d = g_devices[dev];
   if (!d.ready) {
     hipDeviceProp_t prop;
-    int a = 0, b = 0;
+    int blocks = kMaxQueues;
+    auto fits = [&](auto kernel) {
+      int n = 0;
+      if (hipOccupancyMaxActiveBlocksPerMultiprocessor(&n, kernel, kThreads, 0) != hipSuccess) return false;
+      blocks = std::min(blocks, n);
+      return true;
+    };
     void* sym = nullptr;
-    if (hipGetDeviceProperties(&prop, dev) != hipSuccess ||
-        hipOccupancyMaxActiveBlocksPerMultiprocessor(&a, decode_megakernel_hybrid<u16>, kThreads, 0) != hipSuccess ||
-        hipOccupancyMaxActiveBlocksPerMultiprocessor(&b, decode_megakernel_hybrid<float>, kThreads, 0) != hipSuccess ||
-        hipGetSymbolAddress(&sym, HIP_SYMBOL(g_status)) != hipSuccess || hipMemset(sym, 0, sizeof(int32_t) * kStatusWords) != hipSuccess)
+    if (hipGetDeviceProperties(&prop, dev) != hipSuccess || !fits(decode_megakernel_hybrid<u16, false>) || !fits(decode_megakernel_hybrid<float, false>) ||
+        !fits(decode_megakernel_hybrid<u16, true>) || !fits(decode_megakernel_hybrid<float, true>) || hipGetSymbolAddress(&sym, HIP_SYMBOL(g_status)) != hipSuccess || hipMemset(sym, 0, sizeof(int32_t) * kStatusWords) != hipSuccess)
       return QMK_ERR_NO_DEVICE;
-    d.max_queues = std::min(std::min(a, b) * prop.multiProcessorCount, kMaxQueues);
+    d.max_queues = std::min(blocks * prop.multiProcessorCount, kMaxQueues);
     d.status = static_cast<int32_t*>(sym);
     d.ready = true;
   }
@@ -239,7 +247,7 @@ bool layer_pointers(const QmkHybridLayer& l) {
     bool ok = l.in_w && l.o_w && (l.branch > 0 || l.norm1) && (!l.has_mlp || (l.mlp_w && l.down_w)) && (l.branches > 1) == (l.out_norm != nullptr);
     if (l.type == QMK_MIXER_ATTENTION) return ok && l.cache && ((l.rope_cos && l.rope_sin) || l.rot_true == 0);
     ok = ok && l.mid_w && l.mid_b && l.vec0 && l.state;
-    return ok && (l.type == QMK_MIXER_GLA || (l.vec1 && l.vec2 && (l.shift || l.taps == 1)));
+    return ok && (l.type == QMK_MIXER_GLA || (l.gate_w && l.vec1 && l.vec2 && (l.shift || l.taps == 1)));
   }
   bool ok = l.norm1 && l.in_w && l.mid_w && l.vec0;
   if (l.type == QMK_MIXER_LATENT) ok = ok && l.uk_w && l.uv_w && l.rope_cos && l.rope_sin && l.cache;
@@ -285,7 +293,7 @@ size_t decode_buffers(const QmkHybridArgs* a, void* base, DecodeBuffers* b) {
   for (int i = 0; i < a->num_layers; ++i) {
     const QmkHybridLayer& l = a->layers[i];
     if (l.type > QMK_MIXER_DELTA) continue;
-    proj = std::max<size_t>(proj, static_cast<size_t>(l.proj_at) + l.in_rows);
+    proj = std::max<size_t>(proj, static_cast<size_t>(l.proj_at) + l.in_rows + (l.type == QMK_MIXER_DELTA ? l.mix_width : 0));
     mix = std::max<size_t>(mix, std::max(static_cast<size_t>(l.mix_at) + l.mix_width, l.has_mlp ? static_cast<size_t>(l.ff_at) + l.ff : 0));
     if (l.type == QMK_MIXER_ATTENTION) {
       const size_t heads16 = (l.heads + 15) & ~15;
@@ -623,9 +631,13 @@ int prefill_plain(const QmkHybridArgs* a) {
         GemmArgs g = gemm_args(b.h, l.in_w, l.in_rows, D, l, EPI_DELTA_IN);
         g.out = b.q; g.out2 = b.low; g.f0 = b.beta; g.ldo = beta_ld;
         launch_gemm<T, u16, T>(g, st);
-        GemmArgs e = gemm_args(b.low, l.mid_w, l.heads * (l.head_dim + l.v_dim), ranks, l, EPI_DELTA_MID);
-        e.f0 = b.decay; e.out = b.gate;
+        const int keys = l.heads * l.head_dim;
+        GemmArgs e = gemm_args(b.low, l.mid_w, keys, l.rank, l, EPI_DELTA_DECAY);
+        e.lda = ranks; e.f0 = b.decay; e.ldo = keys;
         launch_gemm<T, u16, T>(e, st);
+        GemmArgs f = gemm_args(b.low + l.rank, l.gate_w, W, l.gate_rank, l, EPI_SIGMOID);
+        f.lda = ranks; f.out = b.gate; f.ldo = W;
+        launch_gemm<T, u16, T>(f, st);
         c.raw = b.q; c.beta = b.beta; c.beta_ld = beta_ld; c.values = b.qkv; c.value_ld = W;
         run_chunks<T, true>(a, c, st);
         if (l.taps > 1)
@@ -635,7 +647,7 @@ int prefill_plain(const QmkHybridArgs* a) {
         GemmArgs g = gemm_args(b.h, l.in_w, l.in_rows, D, l, EPI_GLA_IN);
         g.f0 = b.qkv; g.out = b.gate; g.out2 = b.low;
         launch_gemm<T, u16, T>(g, st);
-        GemmArgs e = gemm_args(b.low, l.mid_w, keys, l.rank, l, EPI_GLA_MID);
+        GemmArgs e = gemm_args(b.low, l.mid_w, keys, l.rank, l, EPI_GLA_DECAY);
         e.f0 = b.decay; e.ldo = keys;
         launch_gemm<T, u16, T>(e, st);
         c.qkv = b.qkv; c.values = b.qkv; c.value_ld = 2 * keys + W; c.value_at = 2 * keys;
@@ -709,8 +721,10 @@ extern "C" int qmk_hybrid_decode_step(const QmkHybridArgs* a) {
   p.streams = a->streams; p.vocab = a->vocab; p.vocab_rows = a->vocab_rows; p.slot = a->slot; p.position = a->position; p.flip = a->flip;
   p.max_splits = a->max_splits; p.eps = a->eps; p.logit_scale = a->logit_scale; p.logit_softcap = a->logit_softcap; p.spin_limit = a->spin_limit != 0 ? a->spin_limit : kDefaultSpinLimit;
   const hipStream_t st = static_cast<hipStream_t>(a->stream);
-  if (a->dtype == QMK_HYBRID_F32) hipLaunchKernelGGL(decode_megakernel_hybrid<float>, dim3(a->num_queues), dim3(kThreads), 0, st, p);
-  else hipLaunchKernelGGL(decode_megakernel_hybrid<u16>, dim3(a->num_queues), dim3(kThreads), 0, st, p);
+  auto launch = [&](auto kernel) { hipLaunchKernelGGL(kernel, dim3(a->num_queues), dim3(kThreads), 0, st, p); };
+  const bool plain = a->streams == 0;
+  if (a->dtype == QMK_HYBRID_F32) plain ? launch(decode_megakernel_hybrid<float, true>) : launch(decode_megakernel_hybrid<float, false>);
+  else plain ? launch(decode_megakernel_hybrid<u16, true>) : launch(decode_megakernel_hybrid<u16, false>);
   return hipGetLastError() == hipSuccess ? QMK_OK : QMK_ERR_LAUNCH;
 }
 

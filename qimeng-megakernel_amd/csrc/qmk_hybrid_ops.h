@@ -27,9 +27,10 @@ enum : int {
   OP_OUT_PROJECT = 7,     // output (sub 0) or down (sub 1) projection + all streams of the residual
   OP_UP_GATE = 8,         // norm2 + gate/up rows + gelu
   OP_LM_HEAD = 9,         // final norm + vocabulary rows
-  OP_STATE_STEP = 10,     // gla, delta: decay, recurrence, per-head norm and gate of one head
+  OP_STATE_STEP = 10,     // gla, delta: decays and recurrence of some value columns of one head
   OP_ATTEND_MERGE = 11,   // merge of the parts of one head, output gate
   OP_JOIN = 12,           // rows of [x; embedding] -> x
+  OP_GATE = 13,           // delta: rows of the output gate
 };
 
 constexpr int kMaxStreams = QMK_HYBRID_MAX_STREAMS;
@@ -41,7 +42,8 @@ constexpr int kMaxK = 24576;                  // longest activation vector
 constexpr int kAttendFloats = 33792;          // LDS of the attention op: query, key tile, scores
 constexpr int kMaxRank = 512;
 constexpr int kMaxHeadDim = 256;              // wkv, gla, delta
-constexpr int kStateRows = 32;                // key rows of a head's state a thread holds in registers (gla, delta)
+constexpr int kStateColumns = 64;             // value columns of one OP_STATE_STEP
+constexpr int kStateRows = 32;                // key rows of the state one of its threads holds: 256 rows / (512 / 64) threads a column
 constexpr int kMaxParts = 64;
 constexpr int kDepth = 8;                     // weight rows a wave keeps in flight and reduces together
 constexpr int kAhead = 2;                     // quads of a vector a thread holds in registers (4096 elements a workgroup)
@@ -535,6 +537,34 @@ __device__ __forceinline__ void residual_to_xs(const DecodeParams& p, Smem& s, L
     xs_quad(s, i) = times(xs_quad(s, i), *reinterpret_cast<const float4*>(weight + i), inv);
 }
 
+// What a gla or delta entry left in xs, head by head: RMS norm over the head's values, weight, output gate.
+__device__ __forceinline__ void norm_heads(const DecodeParams& p, Smem& s, LayerRef& l) {
+  const int lane = threadIdx.x & (kWaveSize - 1), wave = threadIdx.x / kWaveSize, n = l.v_dim;
+  const float* gate = p.proj + l.proj_at + (l.type == QMK_MIXER_DELTA ? l.in_rows : 2 * l.heads * l.head_dim + l.mix_width);
+  __syncthreads();
+  constexpr int kPer = kMaxHeadDim / kWaveSize;
+#pragma unroll 1
+  for (int head = wave; head < l.heads; head += kWaves) {
+    float v[kPer], g[kPer], sq = 0.f;
+#pragma unroll
+    for (int j = 0; j < kPer; ++j) {
+      const int i = j * kWaveSize + lane;
+      v[j] = g[j] = 0.f;
+      if (i < n) {
+        v[j] = s.xs[xs_at(head * n + i)];
+        g[j] = ld_shared_f32(gate + head * n + i) * l.vec0[i];
+      }
+      sq = fmaf(v[j], v[j], sq);
+    }
+    const float inv = 1.f / sqrtf(wave_sum(sq) / l.v_true + p.eps);
+#pragma unroll
+    for (int j = 0; j < kPer; ++j) {
+      const int i = j * kWaveSize + lane;
+      if (i < n) s.xs[xs_at(head * n + i)] = v[j] * inv * g[j];
+    }
+  }
+}
+
 // log(1 + e^z) and the decays of the gated recurrences
 __device__ __forceinline__ float softplus(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
 template <class Layer>
@@ -592,41 +622,48 @@ __device__ __forceinline__ bool rows_of(const DecodeParams& p, LayerRef& l, cons
     case OP_OUT_PROJECT:
       if (p.streams > 0 && o.count > kMaxOutRows) return false;
       if (o.sub == 1) return l.has_mlp && o.start + o.count <= D && set(l.down_w, o.start, o.count, l.ff);
-      return o.start + o.count <= D && set(l.o_w, o.start, o.count, l.mix_width);
+      return l.type <= QMK_MIXER_DELTA && o.start + o.count <= D && set(l.o_w, o.start, o.count, l.mix_width);
     case OP_UP_GATE: return l.has_mlp && o.start + o.count <= l.ff && set(l.mlp_w, 2LL * o.start, 2 * o.count, D);
     case OP_STATE_STEP: {
-      if ((l.type != QMK_MIXER_GLA && l.type != QMK_MIXER_DELTA) || o.sub < 0 || o.sub >= l.heads || l.head_dim > kMaxHeadDim || l.v_dim > kMaxHeadDim) return false;
-      const int per = l.type == QMK_MIXER_DELTA ? l.head_dim + l.v_dim : l.head_dim;
-      return set(l.mid_w, static_cast<long long>(o.sub) * per, per, l.rank + l.gate_rank);
+      if ((l.type != QMK_MIXER_GLA && l.type != QMK_MIXER_DELTA) || o.sub < 0 || o.sub >= l.heads || l.head_dim > kMaxHeadDim) return false;
+      return o.count <= kStateColumns && o.start + o.count <= l.v_dim && set(l.mid_w, static_cast<long long>(o.sub) * l.head_dim, l.head_dim, l.rank);
     }
+    case OP_GATE: return l.type == QMK_MIXER_DELTA && o.start + o.count <= l.mix_width && set(l.gate_w, o.start, o.count, l.gate_rank);
     case OP_JOIN: return l.type == QMK_ENTRY_JOIN && o.start + o.count <= D && set(l.in_w, o.start, o.count, 2 * D);
-    case OP_LM_HEAD: return o.start + o.count <= p.vocab_rows && set(p.head, o.start, o.count, D);
+    case OP_LM_HEAD: return (p.streams > 0 || l.type == QMK_ENTRY_FINAL) && o.start + o.count <= p.vocab_rows && set(p.head, o.start, o.count, D);
     default: return false;
   }
 }
 
-template <class T>
+// PLAIN: the kernel of a plain residual (its entries, its ops), which holds none of the other kernel's code, nor that of its.
+template <class T, bool PLAIN>
 __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op& o) {
   LayerRef& l = layer_of(p, o.layer);
+  constexpr bool plain = PLAIN;
+  constexpr unsigned kOps = 1u << OP_IN_PROJECT | 1u << OP_OUT_PROJECT | 1u << OP_UP_GATE | 1u << OP_LM_HEAD |
+                            (plain ? 1u << OP_STATE_STEP | 1u << OP_JOIN | 1u << OP_GATE : 1u << OP_LRU_STEP | 1u << OP_LATENT_ABSORB | 1u << OP_LATENT_VALUE | 1u << OP_WKV_STEP);
+  const int op = o.opcode, type = l.type;
+  if (!(kOps >> op & 1)) return bad_operand(p, o, o.opcode);
+  __builtin_assume(kOps >> op & 1);
+  __builtin_assume(plain ? type >= QMK_MIXER_GLA : type <= QMK_MIXER_WKV);
   Rows m;
   if (!rows_of(p, l, o, m)) return bad_operand(p, o, o.start);
   const int tid = threadIdx.x, D = p.width, S = p.streams;
-  const bool plain = S == 0;
   LayerRef& lead = layer_of(p, o.layer - l.branch);      // the run's first entry
   RowStream g;
   g.start(m.w, m.rows, m.columns);
   clear_part(s, m.rows);
 
   // Asked for ahead of the wait; what the arrays hold depends on the op.  Thread r of the workgroup owns row r.
-  const int op = o.opcode, row = o.start + tid;
+  const int row = o.start + tid;
   const bool mine = tid < m.rows;
   const bool normed = op == OP_IN_PROJECT || op == OP_UP_GATE || op == OP_LM_HEAD;
-  const bool wkv_in = op == OP_IN_PROJECT && l.type == QMK_MIXER_WKV;
+  const bool wkv_in = !plain && op == OP_IN_PROJECT && type == QMK_MIXER_WKV;
   const bool reads_x = plain && (normed || op == OP_JOIN);
   const bool first = !plain && o.layer == 0 && (op == OP_IN_PROJECT || (op == OP_OUT_PROJECT && o.sub == 0));
   const float* norm = plain ? lead.norm1 : op == OP_IN_PROJECT ? l.norm1 : op == OP_UP_GATE ? l.norm2 : p.final_norm;
-  const int channels = l.type == QMK_MIXER_DELTA ? conv_channels(l) : l.mix_width;
-  const size_t shift_copy = l.type == QMK_MIXER_WKV ? static_cast<size_t>(D) : static_cast<size_t>(l.taps - 1) * channels;
+  const int channels = type == QMK_MIXER_DELTA ? conv_channels(l) : l.mix_width;
+  const size_t shift_copy = type == QMK_MIXER_WKV ? static_cast<size_t>(D) : static_cast<size_t>(l.taps - 1) * channels;
   const float* shift_old = l.shift + (static_cast<size_t>(p.slot) * 2 + p.flip) * shift_copy;
   float* shift_new = l.shift + (static_cast<size_t>(p.slot) * 2 + 1 - p.flip) * shift_copy;
   const float* mu = l.vec2 + static_cast<size_t>(o.sub) * D;
@@ -640,9 +677,9 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
     if (wkv_in) {
       load_ahead(w1, shift_old, D);
       load_ahead(w2, mu, D);
-    } else if (op == OP_IN_PROJECT && (l.type == QMK_MIXER_RGLRU || l.type == QMK_MIXER_DELTA) && mine) {
+    } else if (op == OP_IN_PROJECT && type == (plain ? QMK_MIXER_DELTA : QMK_MIXER_RGLRU) && mine) {
       // Everything of the convolution but the current input; the kept inputs move up by one.
-      const bool lru = l.type == QMK_MIXER_RGLRU;
+      constexpr bool lru = !plain;
       const int W = channels, c = lru ? row - W : row;
       if (lru) a[0] = l.in_b[row];
       if (c >= 0 && c < W) {
@@ -657,7 +694,7 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
         a[2] = l.vec2[static_cast<size_t>(l.taps - 1) * W + c];
       }
     }
-  } else if (op == OP_LRU_STEP) {
+  } else if (!plain && op == OP_LRU_STEP) {
     if (mine) {   // rows (r, i) of a channel: neighbouring threads
       const int c = o.sub * l.block_dim + o.start + (tid >> 1);
       state = l.state + static_cast<size_t>(p.slot) * l.mix_width + c;
@@ -665,7 +702,7 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
       a[1] = l.vec0[c];
       a[2] = *state;
     }
-  } else if (op == OP_WKV_STEP) {
+  } else if (!plain && op == OP_WKV_STEP) {
     const int n = l.head_dim, groups = kThreads / n, e = tid % n, group = tid / n;
     state = l.state + (static_cast<size_t>(p.slot) * l.heads + o.sub) * n * n + e;
 #pragma unroll
@@ -677,16 +714,15 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
       const int at = o.sub * n + tid;
       w0[0] = make_float4(l.mid_b[at], l.vec1[at], l.vec0[at], 0.f);
     }
-  } else if (op == OP_STATE_STEP) {
-    const int n = l.v_dim, groups = kThreads / n, e = tid % n, group = tid / n;
-    state = l.state + (static_cast<size_t>(p.slot) * l.heads + o.sub) * l.head_dim * n + e;
+  } else if (plain && op == OP_STATE_STEP) {
+    const int n = o.count, groups = kThreads / n, e = tid % n, group = tid / n;
+    state = l.state + (static_cast<size_t>(p.slot) * l.heads + o.sub) * l.head_dim * l.v_dim + o.start + e;
 #pragma unroll
     for (int j = 0; j < kStateRows; ++j) {
       const int i = group + j * groups;
-      held[j] = group < groups && i < l.head_dim ? state[static_cast<size_t>(i) * n] : 0.f;
+      held[j] = group < groups && i < l.head_dim ? state[static_cast<size_t>(i) * l.v_dim] : 0.f;
     }
-    if (tid < l.head_dim) a[0] = l.mid_b[o.sub * l.head_dim + tid];
-    if (tid < n) a[1] = l.vec0[tid];
+    if (mine) a[0] = l.mid_b[o.sub * l.head_dim + tid];
   } else if (op == OP_OUT_PROJECT && !plain) {
     // Eight lanes per row, one per stream: all streams of the row, the stream's column of the mix, its output weight and
     // its weight in the next sublayer's input.  The streams may be read before the wait: every output projection of a
@@ -712,7 +748,7 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
   if (!wait_stage(p, s, o)) return false;
 
   // The activation vector.
-  if (reads_x) {
+  if (plain && reads_x) {
     residual_to_xs(p, s, lead, normed, op == OP_IN_PROJECT && o.extra, norm, w0);
   } else if (normed) {
     norm_to_xs(p, s, norm, w0, first, l.hc);
@@ -731,7 +767,7 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
       for (int i = (kAhead * kThreads + tid) * 4; i < D; i += kThreads * 4)
         mix(i, *reinterpret_cast<const float4*>(shift_old + i), *reinterpret_cast<const float4*>(mu + i));
     }
-  } else if (op == OP_LATENT_VALUE) {   // merge the parts of this head
+  } else if (!plain && op == OP_LATENT_VALUE) {   // merge the parts of this head
     const int heads16 = (l.heads + 15) & ~15, parts = o.extra;
     const float* from = p.part + static_cast<size_t>(o.sub) * l.rank;
     const int pitch = heads16 * l.rank;
@@ -768,9 +804,9 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
     if (in) s.xs[xs_at(tid)] = acc;
   } else {
     const float* from = p.mix + (op == OP_OUT_PROJECT && o.sub == 1 ? l.ff_at : l.mix_at);
-    if (op == OP_STATE_STEP) {
-      // query, key (unit vectors for the delta rule) and value of the head
-      const bool delta = l.type == QMK_MIXER_DELTA;
+    if (plain && op == OP_STATE_STEP) {
+      // query, key (unit vectors for the delta rule) and values of the head
+      const bool delta = type == QMK_MIXER_DELTA;
       const int n = l.v_dim, dim = l.head_dim, keys = l.kv_heads * dim, kv = o.sub / (l.heads / l.kv_heads);
       const float* proj = p.proj + l.proj_at;
       float q = 0.f, k = 0.f;
@@ -778,10 +814,7 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
         q = ld_shared_f32(proj + kv * dim + tid);
         k = ld_shared_f32(proj + keys + kv * dim + tid);
       }
-      if (tid < n) {
-        s.aux[2 * kMaxHeadDim + tid] = ld_shared_f32(proj + 2 * keys + o.sub * n + tid);
-        if (!delta) a[2] = ld_shared_f32(proj + 2 * keys + (l.heads + o.sub) * n + tid);      // the output gate
-      }
+      if (tid < o.count) s.aux[2 * kMaxHeadDim + tid] = ld_shared_f32(proj + 2 * keys + o.sub * n + o.start + tid);
       from = proj + 2 * keys + l.heads * n * (delta ? 1 : 2);
       if (delta) a[3] = ld_shared_f32(from + l.rank + l.gate_rank + o.sub);      // beta
       if (!delta) q *= l.q_scale;                       // (the projection is left unscaled)
@@ -798,12 +831,14 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
         s.aux[tid] = q;
         s.aux[kMaxHeadDim + tid] = k;
       }
-    } else if (op == OP_LRU_STEP) {
+    } else if (plain && op == OP_GATE) {
+      from = p.proj + l.proj_at + conv_channels(l) + l.rank;
+    } else if (!plain && op == OP_LRU_STEP) {
       if (mine && !(tid & 1)) a[3] = ld_shared_f32(p.proj + o.sub * l.block_dim + o.start + (tid >> 1));
       from = p.proj + l.mix_width + o.sub * l.block_dim;
-    } else if (op == OP_LATENT_ABSORB) {
+    } else if (!plain && op == OP_LATENT_ABSORB) {
       from = p.proj + o.sub * l.q_stride;
-    } else if (op == OP_WKV_STEP) {
+    } else if (!plain && op == OP_WKV_STEP) {
       const int n = l.head_dim, N = l.heads * n, at = o.sub * n + tid;
       if (mine) {
         const float r = ld_shared_f32(p.proj + at), k = ld_shared_f32(p.proj + N + at), v = ld_shared_f32(p.proj + 2 * N + at);
@@ -816,6 +851,7 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
       from = p.proj + 4 * N;
     }
     load_vector(s, from, m.columns);
+    if (plain && op == OP_OUT_PROJECT && o.sub == 0 && l.type != QMK_MIXER_ATTENTION) norm_heads(p, s, l);
   }
   __syncthreads();
   stamp(p, s, 1);
@@ -826,7 +862,7 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
   // What happens to the rows' sums; a pair of rows is a pair of lanes.
   float t = mine && (plain || op != OP_OUT_PROJECT) ? row_total(s, tid) : 0.f;
   static_assert(kMaxRows <= kThreads && kMaxStreams == 8, "one row per thread, eight values ahead");
-  if (op == OP_JOIN) {
+  if (plain && op == OP_JOIN) {
     if (mine) st_shared_f32(p.x + static_cast<size_t>(l.x_to) * D + row, t);
   } else if (op == OP_OUT_PROJECT && plain) {
     if (mine) st_shared_f32(p.out + static_cast<size_t>(o.sub == 1 ? QMK_HYBRID_MAX_BRANCHES : l.branch) * D + row, t);
@@ -848,7 +884,7 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
     if (mine) {
       const int W = l.mix_width;
       int gate = 0;          // 1: sigmoid, 2: times sigmoid (silu), 3: gelu
-      if (l.type == QMK_MIXER_RGLRU) {
+      if (!plain && type == QMK_MIXER_RGLRU) {
         t += a[0];
         if (row < W) {
           gate = 3;
@@ -856,7 +892,7 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
           if (l.taps > 1) shift_new[static_cast<size_t>(l.taps - 2) * W + row - W] = t;
           t = fmaf(a[2], t, a[1]);
         }
-      } else if (l.type == QMK_MIXER_LATENT) {
+      } else if (!plain && type == QMK_MIXER_LATENT) {
         const int q_rows = l.heads * l.q_stride, g_rows = l.heads * l.v_dim;
         int d = -1;
         if (row < q_rows) d = row % l.q_stride - l.head_dim;
@@ -867,7 +903,7 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
           const float c = l.rope_cos[at], sn = l.rope_sin[at];
           t = t * c + ((tid & 1) ? pair * sn : -(pair * sn));
         }
-      } else if (l.type == QMK_MIXER_ATTENTION) {
+      } else if (plain && type == QMK_MIXER_ATTENTION) {
         const int q_rows = l.heads * l.q_stride, k_rows = l.kv_heads * l.head_dim, v_rows = l.kv_heads * l.v_dim;
         const int d = row < q_rows ? row % l.q_stride : row < q_rows + k_rows ? (row - q_rows) % l.head_dim : l.rot_true;
         if (d < l.rot_true) {
@@ -876,7 +912,7 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
           t = t * c + ((tid & 1) ? pair * sn : -(pair * sn));
         }
         if (row >= q_rows + k_rows + v_rows) gate = 1;
-      } else if (l.type == QMK_MIXER_DELTA) {
+      } else if (plain && type == QMK_MIXER_DELTA) {
         if (row < channels) {
           if (l.taps > 1) shift_new[static_cast<size_t>(l.taps - 2) * channels + row] = t;
           t = fmaf(a[2], t, a[1]);
@@ -884,12 +920,12 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
         } else if (row >= channels + l.rank + l.gate_rank) {
           gate = 1;
         }
-      } else if (l.type == QMK_MIXER_GLA) {
+      } else if (plain && type == QMK_MIXER_GLA) {
         const int from = 2 * l.heads * l.head_dim + l.heads * l.v_dim;
         if (row >= from && row < from + l.heads * l.v_dim) gate = 2;
-      } else if (row >= 4 * W) {
+      } else if (!plain && row >= 4 * W) {
         t = tanhf(t);
-      } else if (row >= 3 * W) {
+      } else if (!plain && row >= 3 * W) {
         gate = 2;
       }
       if (gate) {
@@ -899,7 +935,7 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
       }
       st_shared_f32(p.proj + l.proj_at + row, t);
     }
-  } else if (op == OP_LRU_STEP) {
+  } else if (!plain && op == OP_LRU_STEP) {
     const float gate = sigmoid(t + a[0]), in_gate = dpp_f32<kDppQuadXor1>(0.f, gate);
     if (mine && !(tid & 1)) {
       const int c = o.start + (tid >> 1);
@@ -909,9 +945,9 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
       *state = now;
       st_shared_f32(p.mix + o.sub * l.block_dim + c, now * a[3]);
     }
-  } else if (op == OP_LATENT_VALUE) {
+  } else if (!plain && op == OP_LATENT_VALUE) {
     if (mine) st_shared_f32(p.mix + o.sub * l.v_dim + row, t * a[0]);
-  } else if (op == OP_LATENT_ABSORB) {
+  } else if (!plain && op == OP_LATENT_ABSORB) {
     if (mine) st_shared_f32(p.absorbed + o.sub * l.rank + row, t);
     if (o.extra) {   // the step's cache row: normed latent, rotated key part
       const float* c = p.proj + l.heads * (l.q_stride + l.v_dim);
@@ -935,7 +971,7 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
         put(i < l.rot_dim ? l.rank + i : width, i < l.rot_dim ? ld_shared_f32(c + l.rank + i) : 0.f);
       }
     }
-  } else if (op == OP_WKV_STEP) {
+  } else if (!plain && op == OP_WKV_STEP) {
     const int n = l.head_dim, groups = kThreads / n, e = tid % n, group = tid / n;
     const float *r = s.aux, *k = r + kMaxHeadDim, *v = k + kMaxHeadDim, *w = v + kMaxHeadDim, *u = w + kMaxHeadDim;
     if (mine) s.aux[3 * kMaxHeadDim + tid] = expf(-expf(t + w0[0].x));
@@ -963,14 +999,13 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
     const float sq = block_sum(val * val, s.scratch);   // storage columns behind the true head size hold zeros
     const float inv = 1.f / sqrtf(sq / l.head_dim_true + p.eps);
     if (mine) st_shared_f32(p.mix + o.sub * n + tid, val * inv * w0[0].z * w0[0].w);
-  } else if (op == OP_STATE_STEP) {
+  } else if (plain && op == OP_STATE_STEP) {
     // S <- decay S, u = beta (v - S^T k), S <- S + k u^T, o = S^T q, with S^T k and S^T q taken together:
     // o = (decay S)^T q + (q . k) u.  Without the delta rule u = v.
-    const bool delta = l.type == QMK_MIXER_DELTA;
-    const int n = l.v_dim, dim = l.head_dim, groups = kThreads / n, e = tid % n, group = tid / n;
-    float *q = s.aux, *k = q + kMaxHeadDim, *v = k + kMaxHeadDim, *w = v + kMaxHeadDim, *gate = w + kMaxHeadDim;
-    if (tid < dim) w[tid] = delta ? delta_decay(l, o.sub, t + a[0]) : gla_decay(l, t + a[0]);
-    else if (mine) gate[tid - dim] = sigmoid(t);
+    const bool delta = type == QMK_MIXER_DELTA;
+    const int n = o.count, dim = l.head_dim, groups = kThreads / n, e = tid % n, group = tid / n;
+    float *q = s.aux, *k = q + kMaxHeadDim, *v = k + kMaxHeadDim, *w = v + kMaxHeadDim;
+    if (mine) w[tid] = delta ? delta_decay(l, o.sub, t + a[0]) : gla_decay(l, t + a[0]);
     __syncthreads();
     float ak = 0.f, aq = 0.f;
     if (group < groups) {
@@ -982,12 +1017,6 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
           ak = fmaf(k[i], held[j], ak);
           aq = fmaf(q[i], held[j], aq);
         }
-      }
-#pragma unroll 1
-      for (int i = group + kStateRows * groups; i < dim; i += groups) {
-        const float h = w[i] * state[static_cast<size_t>(i) * n];
-        ak = fmaf(k[i], h, ak);
-        aq = fmaf(q[i], h, aq);
       }
       s.xs[group * n + e] = ak;
       s.xs[(groups + group) * n + e] = aq;
@@ -1004,15 +1033,12 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
 #pragma unroll
       for (int j = 0; j < kStateRows; ++j) {
         const int i = group + j * groups;
-        if (i < dim) state[static_cast<size_t>(i) * n] = fmaf(k[i], u, held[j]);
+        if (i < dim) state[static_cast<size_t>(i) * l.v_dim] = fmaf(k[i], u, held[j]);
       }
-#pragma unroll 1
-      for (int i = group + kStateRows * groups; i < dim; i += groups)
-        state[static_cast<size_t>(i) * n] = fmaf(k[i], u, w[i] * state[static_cast<size_t>(i) * n]);
     }
-    const float val = tid < n ? fmaf(a[4], u, aq) : 0.f;
-    const float inv = 1.f / sqrtf(block_sum(val * val, s.scratch) / l.v_true + p.eps);
-    if (tid < n) st_shared_f32(p.mix + l.mix_at + o.sub * n + tid, val * inv * a[1] * (delta ? gate[tid] : a[2]));
+    if (tid < n) st_shared_f32(p.mix + l.mix_at + o.sub * l.v_dim + o.start + tid, fmaf(a[4], u, aq));
+  } else if (plain && op == OP_GATE) {
+    if (mine) st_shared_f32(p.proj + l.proj_at + l.in_rows + row, sigmoid(t));
   } else {   // OP_LM_HEAD
     if (plain) t = soft_cap(t * p.logit_scale, p.logit_softcap);
     if (mine) p.logits[row] = t;
@@ -1092,14 +1118,14 @@ __host__ __device__ constexpr int attend_floats(int row_elements, int element_by
 // Latent: heads [16 sub, 16 sub + 16), a row is [latent | rotated key], the latent is the value.  Attention: the heads of key
 // head g = sub / b, sixteen of them from 16 (sub % b) on, b = ceil(heads per key head / 16); a row is g's [key | value], and
 // the step's own row comes from the projections (one instruction per key head puts it into the cache).
-template <class T>
+template <class T, bool PLAIN>
 __device__ __forceinline__ bool op_attend(const DecodeParams& p, Smem& s, const Op& o) {
   constexpr int kKeys = attend_keys(sizeof(T)), kTiles = kKeys / 16, kSlices = kWaves / kTiles, kPer = kKeys * 16 / kThreads, kSp = kKeys + 8;
   constexpr int kUnit = 16 / sizeof(T);
   LayerRef& l = layer_of(p, o.layer);
   const int heads16 = (l.heads + 15) & ~15;
-  const bool latent = l.type == QMK_MIXER_LATENT;
-  if ((!latent && l.type != QMK_MIXER_ATTENTION) || o.sub < 0 || o.start < 0 || o.count <= 0 || o.count > p.max_splits || o.start >= o.count || o.extra < 0)
+  constexpr bool latent = !PLAIN;
+  if (l.type != (latent ? QMK_MIXER_LATENT : QMK_MIXER_ATTENTION) || o.sub < 0 || o.start < 0 || o.count <= 0 || o.count > p.max_splits || o.start >= o.count || o.extra < 0)
     return bad_operand(p, o, o.start);
   const int group = latent ? l.heads : l.heads / l.kv_heads, blocks = (group + 15) / 16, kv = o.sub / blocks, block = o.sub % blocks;
   const int values = latent ? l.rank : l.v_dim, value_at = latent ? 0 : l.head_dim;      // columns of a row that are its value

@@ -153,57 +153,81 @@ __global__ __launch_bounds__(kPfThreads) void chunk_prepare(const ChunkArgs g) {
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int kv = head / (l.heads / l.kv_heads), keys = l.kv_heads * dim;
 
-  auto convolved = [&](int t, int c) {     // token m0 + t, channel c
-    const int W = conv_channels(l), taps = l.taps;
-    const T* x = static_cast<const T*>(g.raw);
-    const float* old = l.shift + (static_cast<size_t>(g.slot) * 2 + g.flip) * (taps - 1) * W;
-    float acc = 0.f;
-    for (int j = 0; j < taps; ++j) {
-      const int at = m0 + t - (taps - 1) + j;
-      acc = fmaf(l.vec2[static_cast<size_t>(j) * W + c], at >= 0 ? to_f32(x[static_cast<size_t>(at) * W + c]) : old[static_cast<size_t>(at + taps - 1) * W + c], acc);
-    }
-    return acc * sigmoid(acc);
-  };
-  for (int t = wave; t < C; t += kChunkWaves) {
-    const bool real = t < count;
-    float q[kMaxHeadDim / 64], k[kMaxHeadDim / 64], nq = 0.f, nk = 0.f;
+  // A thread takes a channel of q, k or v down the chunk's tokens.
+  for (int id = tid; id < (DELTA ? 2 * dim + n : 2 * dim); id += kPfThreads) {
+    const int part = id / dim < 2 ? id / dim : 2, c = id - part * dim;
+    float v[C];
+    if constexpr (DELTA) {
+      const int W = conv_channels(l), taps = l.taps, ch = part == 0 ? kv * dim + c : part == 1 ? keys + kv * dim + c : 2 * keys + head * n + c;
+      const T* x = static_cast<const T*>(g.raw) + ch;
+      const float* old = l.shift + (static_cast<size_t>(g.slot) * 2 + g.flip) * (taps - 1) * W + ch;
+      const float* weight = l.vec2 + ch;
+      auto input = [&](int at) {      // token at of the portion; tokens behind it are not used
+        return at >= 0 ? to_f32(x[static_cast<size_t>(min(at, g.M - 1)) * W]) : old[static_cast<size_t>(at + taps - 1) * W];
+      };
+      constexpr int kFew = 4;
+      if (taps <= kFew) {
+        float in[C + kFew - 1], w[kFew];
 #pragma unroll
-    for (int j = 0; j < kMaxHeadDim / 64; ++j) {
-      const int c = j * 64 + lane;
-      q[j] = k[j] = 0.f;
-      if (real && c < dim) {
-        if constexpr (DELTA) {
-          q[j] = convolved(t, kv * dim + c);
-          k[j] = convolved(t, keys + kv * dim + c);
-        } else {
-          const float* row = g.qkv + static_cast<size_t>(m0 + t) * (2 * keys + l.heads * n);
-          q[j] = row[kv * dim + c];
-          k[j] = row[keys + kv * dim + c];
+        for (int j = 0; j < kFew; ++j) w[j] = j >= kFew - taps ? weight[static_cast<size_t>(j - kFew + taps) * W] : 0.f;
+#pragma unroll
+        for (int j = 0; j < C + kFew - 1; ++j) in[j] = j >= kFew - taps ? input(m0 - (kFew - 1) + j) : 0.f;
+#pragma unroll
+        for (int t = 0; t < C; ++t) {
+          v[t] = 0.f;
+#pragma unroll
+          for (int j = 0; j < kFew; ++j) v[t] = fmaf(w[j], in[t + j], v[t]);
+        }
+      } else {
+#pragma unroll
+        for (int t = 0; t < C; ++t) {
+          v[t] = 0.f;
+          for (int j = 0; j < taps; ++j) v[t] = fmaf(weight[static_cast<size_t>(j) * W], input(m0 + t - (taps - 1) + j), v[t]);
         }
       }
-      nq = fmaf(q[j], q[j], nq);
-      nk = fmaf(k[j], k[j], nk);
-    }
-    float iq = l.q_scale, ik = 1.f;
-    if constexpr (DELTA) {
-      iq = l.q_scale / sqrtf(wave_sum(nq) + 1e-6f);
-      ik = 1.f / sqrtf(wave_sum(nk) + 1e-6f);
-    }
 #pragma unroll
-    for (int j = 0; j < kMaxHeadDim / 64; ++j) {
-      const int c = j * 64 + lane;
-      if (c < dim) {
-        sq[t][c] = q[j] * iq;
-        sk[t][c] = k[j] * ik;
-        sg[t][c] = real ? g.decay[static_cast<size_t>(m0 + t) * l.heads * dim + head * dim + c] : 1.f;
+      for (int t = 0; t < C; ++t) v[t] *= sigmoid(v[t]);
+      if (part == 2) {
+        float* to = g.values + static_cast<size_t>(m0) * g.value_ld + g.value_at + head * n + c;
+#pragma unroll
+        for (int t = 0; t < C; ++t)
+          if (t < count) to[static_cast<size_t>(t) * g.value_ld] = v[t];
+        continue;
       }
+    } else {
+      const int ld = 2 * keys + l.heads * n;
+      const float* row = g.qkv + static_cast<size_t>(m0) * ld + part * keys + kv * dim + c;
+#pragma unroll
+      for (int t = 0; t < C; ++t) v[t] = row[static_cast<size_t>(min(t, count - 1)) * ld] * (part == 0 ? l.q_scale : 1.f);
     }
-    if constexpr (DELTA) {
-      if (real)
-        for (int c = lane; c < n; c += 64) g.values[static_cast<size_t>(m0 + t) * g.value_ld + g.value_at + head * n + c] = convolved(t, 2 * keys + head * n + c);
-    }
+    auto& to = part == 0 ? sq : sk;
+#pragma unroll
+    for (int t = 0; t < C; ++t) to[t][c] = t < count ? v[t] : 0.f;
+  }
+  for (int c = tid; c < dim; c += kPfThreads) {
+    const float* row = g.decay + static_cast<size_t>(m0) * l.heads * dim + head * dim + c;
+    float v[C];
+#pragma unroll
+    for (int t = 0; t < C; ++t) v[t] = row[static_cast<size_t>(min(t, count - 1)) * l.heads * dim];
+#pragma unroll
+    for (int t = 0; t < C; ++t) sg[t][c] = t < count ? v[t] : 1.f;
   }
   __syncthreads();
+  if constexpr (DELTA) {      // unit vectors
+    for (int t = wave; t < C; t += kChunkWaves) {
+      float nq = 0.f, nk = 0.f;
+      for (int c = lane; c < dim; c += 64) {
+        nq = fmaf(sq[t][c], sq[t][c], nq);
+        nk = fmaf(sk[t][c], sk[t][c], nk);
+      }
+      const float iq = l.q_scale / sqrtf(wave_sum(nq) + 1e-6f), ik = 1.f / sqrtf(wave_sum(nk) + 1e-6f);
+      for (int c = lane; c < dim; c += 64) {
+        sq[t][c] *= iq;
+        sk[t][c] *= ik;
+      }
+    }
+    __syncthreads();
+  }
 
   float* rec = g.chunks + (static_cast<size_t>(chunk) * l.heads + head) * chunk_floats(dim);
   const int tiles = dim / 16;
@@ -296,6 +320,7 @@ __global__ __launch_bounds__(kPfThreads) void keep_inputs(const T* x, QmkHybridL
 // between a tile's last product and the first use of its result on the path that skips the next tile.
 template <int TILES, bool DELTA>
 __global__ __launch_bounds__(kChunkWaves * 64) void chunk_scan(const ChunkArgs g) {
+  constexpr int kAhead = TILES <= 2 ? 4 : 2;      // chunks in flight
   __shared__ f32x4 px[2][kChunkWaves][64], po[2][kChunkWaves][64];
   const QmkHybridLayer& l = g.layer;
   const int dim = l.head_dim, n = l.v_dim, head = blockIdx.x, v0 = blockIdx.y * 16, tiles = dim / 16;
@@ -341,8 +366,7 @@ __global__ __launch_bounds__(kChunkWaves * 64) void chunk_scan(const ChunkArgs g
     for (int i = 0; i < 4; ++i) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], b[i], c, 0, 0, 0);
     return c;
   };
-  auto advance = [&](Fragments& f, Fragments& next, int chunk) {
-    if (chunk + 1 < chunks) fetch(next, chunk + 1);
+  auto advance = [&](Fragments& f, int chunk) {      // ... and the fragments' place is filled again
     const int buf = chunk & 1;
     f32x4 x = {}, o = {};
     if constexpr (DELTA) {
@@ -372,12 +396,16 @@ __global__ __launch_bounds__(kChunkWaves * 64) void chunk_scan(const ChunkArgs g
         if (m < g.M) g.out[static_cast<size_t>(m) * l.heads * n + head * n + v0 + col] = o[i];
       }
     }
+    if (chunk + kAhead < chunks) fetch(f, chunk + kAhead);
   };
-  Fragments even, odd;
-  fetch(even, 0);
-  for (int chunk = 0; chunk < chunks; chunk += 2) {
-    advance(even, odd, chunk);
-    if (chunk + 1 < chunks) advance(odd, even, chunk + 1);
+  Fragments f[kAhead];
+#pragma unroll
+  for (int a = 0; a < kAhead; ++a)
+    if (a < chunks) fetch(f[a], a);
+  for (int chunk = 0; chunk < chunks; chunk += kAhead) {
+#pragma unroll
+    for (int a = 0; a < kAhead; ++a)
+      if (chunk + a < chunks) advance(f[a], chunk + a);
   }
 #pragma unroll
   for (int j = 0; j < TILES; ++j)

@@ -26,9 +26,10 @@ enum : int {
   EPI_ADD,              // onto the fp32 residual
   EPI_ATTENTION_IN,     // rotation of q and k, k and v into the cache, sigmoid of the gate
   EPI_DELTA_IN,         // raw q, k, v; raw ranks; sigmoid of the step sizes
-  EPI_DELTA_MID,        // decays and output gate
+  EPI_DELTA_DECAY,
+  EPI_SIGMOID,
   EPI_GLA_IN,           // q, k, v fp32; silu gate; raw rank
-  EPI_GLA_MID,          // decays
+  EPI_GLA_DECAY,
 };
 
 struct GemmArgs {
@@ -223,18 +224,17 @@ __device__ __forceinline__ void epilogue(const GemmArgs& g, int group, int m, in
       }
       break;
     }
-    case EPI_DELTA_MID: {
-      const int per = l.head_dim + l.v_dim, head = n / per, c = n % per;
-      if (c < l.head_dim) {
-        const f32x4 b = *reinterpret_cast<const f32x4*>(l.mid_b + head * l.head_dim + c);
+    case EPI_DELTA_DECAY: {
+      const f32x4 b = *reinterpret_cast<const f32x4*>(l.mid_b + n);
 #pragma unroll
-        for (int i = 0; i < 4; ++i) v[i] = delta_decay(l, head, v[i] + b[i]);
-        store4(g.f0 + static_cast<size_t>(m) * l.heads * l.head_dim + head * l.head_dim + c, v);
-      } else {
+      for (int i = 0; i < 4; ++i) v[i] = delta_decay(l, n / l.head_dim, v[i] + b[i]);
+      store4(g.f0 + static_cast<size_t>(m) * g.ldo + n, v);
+      break;
+    }
+    case EPI_SIGMOID: {
 #pragma unroll
-        for (int i = 0; i < 4; ++i) v[i] = sigmoid(v[i]);
-        store4(static_cast<T*>(g.out) + static_cast<size_t>(m) * l.mix_width + head * l.v_dim + c - l.head_dim, v);
-      }
+      for (int i = 0; i < 4; ++i) v[i] = sigmoid(v[i]);
+      store4(static_cast<T*>(g.out) + static_cast<size_t>(m) * g.ldo + n, v);
       break;
     }
     case EPI_GLA_IN: {
@@ -250,7 +250,7 @@ __device__ __forceinline__ void epilogue(const GemmArgs& g, int group, int m, in
       }
       break;
     }
-    case EPI_GLA_MID: {
+    case EPI_GLA_DECAY: {
       const f32x4 b = *reinterpret_cast<const f32x4*>(l.mid_b + n);
 #pragma unroll
       for (int i = 0; i < 4; ++i) v[i] = gla_decay(l, v[i] + b[i]);
@@ -620,7 +620,7 @@ __global__ __launch_bounds__(kPfThreads) void window_attention(const T* q, Keys<
   __shared__ __align__(16) T sk[kKeys][QT * 32 + kPadK];
   __shared__ __align__(16) T sv[VT * 16][kKeys + kPadV];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g = lane >> 4, col = lane & 15;
-  const int head = blockIdx.y, kv = head / keys.heads_per, q0 = blockIdx.x * 64;
+  const int head = blockIdx.y, kv = head / keys.heads_per, q0 = (gridDim.x - 1 - blockIdx.x) * 64;      // the longest rows of keys first
   const int dq = l.q_stride, steps = dq / 32, vt = l.v_dim / 16, width = l.rank + l.rot_dim;
   const int m = q0 + wave * 16 + col, pos = position + m;
   Frag<T> fq[QT];

@@ -88,7 +88,8 @@ class RMS_LMHead(StageInstruction):
 
 @dataclass
 class GatedStateStep(StageInstruction):
-    """One head of a gated linear attention or gated delta rule: decay, recurrence, per-head norm and gate."""
+    """Value columns ``start`` .. of one head of a gated linear attention or gated delta rule: decays and recurrence.  The
+    output projection norms the head and applies the gate."""
     OPCODE: ClassVar[int] = 10
 
 
@@ -104,5 +105,11 @@ class JoinProject(StageInstruction):
     OPCODE: ClassVar[int] = 12
 
 
+@dataclass
+class OutputGate(StageInstruction):
+    """Rows of a low-rank output gate."""
+    OPCODE: ClassVar[int] = 13
+
+
 INSTRUCTIONS = {c.OPCODE: c for c in (NoOp, RMS_InProject, GatedRecurrence, LatentAbsorb, AttendSplitKV, LatentValue, WkvStep,
-                                      OutProject_Streams, RMS_UpGate_Gelu, RMS_LMHead, GatedStateStep, AttendMerge, JoinProject)}
+                                      OutProject_Streams, RMS_UpGate_Gelu, RMS_LMHead, GatedStateStep, AttendMerge, JoinProject, OutputGate)}

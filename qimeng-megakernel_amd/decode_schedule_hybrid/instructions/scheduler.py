@@ -2,9 +2,9 @@
 
 A layer on residual streams is a chain of stages: input projections, the mixer's middle (recurrence; absorb, attend, value;
 wkv step), output projection, and for a feed-forward up/gate and down.  A layer run on the plain residual, whose branches and
-feed-forward read the same input, is three or four stages: all input projections and up/gate; state steps and attention;
-merges, the output projections of the state branches and down; the output projections of the attention.  (Without an
-attention the down projection runs beside the state steps, and the output projections follow.)  What a run leaves is added by
+feed-forward read the same input, is three or four stages: all input projections and up/gate; state steps, attention and
+low-rank output gates; merges, the output projections of the state branches and down; the output projections of the
+attention.  (Without an attention the down projection runs beside the state steps, and the output projections follow.)  What a run leaves is added by
 the stage that reads the residual next.  The LM head ends the step.  Each stage's output rows are cut into
 blocks of equal size, about one per queue, and dealt to the queues from queue 0 on (the leaders of the per-XCD waits are
 the first eight queues, so they take part in every stage).  All output and down projections are cut alike: a queue owns its
@@ -28,7 +28,8 @@ MAX_OUT_ROWS = 64          # ... of an output projection: a thread per row and s
 MIN_ROWS = 4
 KEYS_PER_PART = 64
 MAX_PARTS = 32
-ATTEND_COLUMNS = 128       # latent columns one attention instruction sums up
+ATTEND_COLUMNS = 128       # latent or value columns one attention instruction sums up
+STATE_COLUMNS = 64         # value columns of one state step: all key rows fit its threads' registers
 BARRIER_ROWS, BARRIER_SLOTS = 54, 48
 
 
@@ -108,6 +109,7 @@ class HybridScheduler:
         stages[0][0].extra = 1
         steps: list[D.StageInstruction] = []
         merges: list[D.StageInstruction] = []
+        gates: list[tuple[int, Any]] = []
         early: list[tuple[int, Any]] = []
         late: list[tuple[int, Any]] = []
         for i, l in branches.items():
@@ -119,12 +121,14 @@ class HybridScheduler:
                 merges += [D.AttendMerge(i, h, 0, parts) for h in range(l.heads)]
                 late.append(out)
             else:
-                steps = [D.GatedStateStep(i, h, 0, 1) for h in range(l.heads)] + steps
+                steps = [D.GatedStateStep(i, h, a, min(STATE_COLUMNS, l.v_s - a)) for h in range(l.heads) for a in range(0, l.v_s, STATE_COLUMNS)] + steps
+                if l.gate_rank:
+                    gates.append((l.mix_width, lambda a, n, i=i: D.OutputGate(i, 0, a, n)))
                 early.append(out)
         if merges:
-            stages += [steps, merges + self._spread(early + down, len(merges)), self._spread(late)]
+            stages += [steps + self._spread(gates, len(steps)), merges + self._spread(early + down, len(merges)), self._spread(late)]
         else:
-            stages += [steps + (self._spread(down, len(steps)) if down else []), self._spread(early)]
+            stages += [steps + self._spread(gates + down, len(steps)), self._spread(early)]
         return stages
 
     def stages(self) -> list[list[D.StageInstruction]]:

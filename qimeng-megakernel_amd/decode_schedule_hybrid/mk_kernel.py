@@ -25,7 +25,7 @@ _ERRORS = {1: "null argument", 2: "struct_size does not match the library", 3: "
            34: "device: counter wait ran out of polls"}
 
 #: pointer fields of the layer table = keys of a layer's weight and state tensors
-_LAYER_POINTERS = ("norm1", "norm2", "in_w", "in_b", "mid_w", "mid_b", "uk_w", "uv_w", "o_w", "mlp_w", "down_w", "vec0", "vec1", "vec2", "rope_cos",
+_LAYER_POINTERS = ("norm1", "norm2", "in_w", "in_b", "mid_w", "mid_b", "gate_w", "uk_w", "uv_w", "o_w", "mlp_w", "down_w", "vec0", "vec1", "vec2", "rope_cos",
                    "rope_sin", "hc", "next1", "next2", "out_norm", "cache", "state", "shift")
 
 
@@ -90,7 +90,7 @@ def layer_table(globs: Globals) -> ctypes.Array:
             e.proj_at, e.mix_at = proj_at, mix_at
         if l.type not in ("join", "final"):
             e.in_rows, e.mix_width, e.heads, e.kv_heads = l.in_rows, l.mix_width, l.heads, l.kv_heads
-            proj_at, mix_at = proj_at + l.in_rows, mix_at + l.mix_width
+            proj_at, mix_at = proj_at + l.in_rows + (l.mix_width if l.type == "delta" else 0), mix_at + l.mix_width
         if entry.ff and globs.shape.plain:
             e.ff_at = sum(b.shape.mix_width for b in entries[i : i + entry.branches])
         if l.type == "latent_attention":

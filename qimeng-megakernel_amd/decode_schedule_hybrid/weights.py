@@ -205,8 +205,8 @@ def _pack_delta(l: LayerShape, Ds: int, raw, p: dict[str, Tensor]) -> None:
     parts = (("q", G, l.dim_s), ("k", G, l.dim_s), ("v", H, l.v_s))
     p["in_w"] = torch.cat([_rows(raw(name), n, size, Ds) for name, n, size in parts]
                           + [_pad(raw("a1"), l.rank_s, Ds), _pad(raw("g1"), l.gate_rank_s, Ds), _pad(raw("b"), l.heads_s, Ds)])
-    decay, gate = _pad(raw("a2").reshape(H, l.dim, -1), H, l.dim_s, l.rank_s), _pad(raw("g2").reshape(H, l.v_dim, -1), H, l.v_s, l.gate_rank_s)
-    p["mid_w"] = torch.cat([F.pad(decay, (0, l.gate_rank_s)), F.pad(gate, (l.rank_s, 0))], dim=1).reshape(H * (l.dim_s + l.v_s), l.rank_s + l.gate_rank_s)
+    p["mid_w"] = _rows(raw("a2"), H, l.dim_s, l.rank_s)
+    p["gate_w"] = _rows(raw("g2"), H, l.v_s, l.gate_rank_s)
     p["mid_b"] = _vector(raw("dt_bias"), H, l.dim_s)
     p["vec0"] = _pad(raw("norm").float(), l.v_s)
     p["vec1"] = _pad(-torch.exp(raw("A_log").double()).float(), l.heads_s)
