@@ -456,6 +456,7 @@ void launch_attention(const QmkHybridArgs* a, const QmkHybridLayer& l, const T* 
     hipLaunchKernelGGL(kernel, dim3((a->tokens + 63) / 64, l.heads), dim3(kPfThreads), 0, st, q, keys, rows, vt, gate, l, first, a->position, a->tokens, cap, out);
   };
   if (l.q_stride <= 128 && l.v_dim <= 64) launch(window_attention<T, 4, 4>);
+  else if (l.q_stride <= 128 && l.v_dim <= 128) launch(window_attention<T, 4, 8>);
   else if (l.q_stride <= 192 && l.v_dim <= 128) launch(window_attention<T, 6, 8>);
   else launch(window_attention<T, 8, 16>);
 }
@@ -555,11 +556,11 @@ int prefill(const QmkHybridArgs* a) {
 template <class T, bool DELTA>
 void run_chunks(const QmkHybridArgs* a, const ChunkArgs& g, hipStream_t st) {
   const QmkHybridLayer& l = g.layer;
-  const int chunks = (g.M + kChunkTokens - 1) / kChunkTokens, tiles = l.head_dim / 16;
+  const int chunks = (g.M + kChunkTokens - 1) / kChunkTokens, tiles = wave_tiles(l.head_dim);
   hipLaunchKernelGGL((chunk_prepare<T, DELTA>), dim3(chunks, l.heads), dim3(kPfThreads), 0, st, g);
   const dim3 grid(l.heads, l.v_dim / 16), block(kChunkWaves * 64);
-  if (tiles <= kChunkWaves) hipLaunchKernelGGL((chunk_scan<1, DELTA>), grid, block, 0, st, g);
-  else if (tiles <= 2 * kChunkWaves) hipLaunchKernelGGL((chunk_scan<2, DELTA>), grid, block, 0, st, g);
+  if (tiles == 1) hipLaunchKernelGGL((chunk_scan<1, DELTA>), grid, block, 0, st, g);
+  else if (tiles == 2) hipLaunchKernelGGL((chunk_scan<2, DELTA>), grid, block, 0, st, g);
   else hipLaunchKernelGGL((chunk_scan<4, DELTA>), grid, block, 0, st, g);
 }
 

@@ -126,9 +126,12 @@ __global__ __launch_bounds__(kPfThreads) void transpose_values(const T* cache, i
 constexpr int kChunkTokens = 16;
 constexpr int kChunkWaves = 4;
 
-// Floats of one (chunk, head): per tile of sixteen key channels the fragments of G q, G k and D k and the decays G over the
-// whole chunk, then B and T.  A fragment is in the order the matrix instruction takes it: [lane][4].
-__host__ __device__ inline int chunk_floats(int head_dim) { return head_dim / 16 * (3 * 256 + 16) + 2 * 256; }
+// Tiles of sixteen key channels a wave of chunk_scan holds, and those of a head, the last ones zeros.
+__host__ __device__ constexpr int wave_tiles(int head_dim) { return head_dim <= 64 ? 1 : head_dim <= 128 ? 2 : 4; }
+__host__ __device__ constexpr int chunk_tiles(int head_dim) { return wave_tiles(head_dim) * kChunkWaves; }
+// Floats of one (chunk, head): per tile the fragments of G q, G k and D k and the decays G over the whole chunk, then B and
+// T.  A fragment is in the order the matrix instruction takes it: [lane][4].
+__host__ __device__ constexpr int chunk_floats(int head_dim) { return chunk_tiles(head_dim) * (3 * 256 + 16) + 2 * 256; }
 
 struct ChunkArgs {
   QmkHybridLayer layer;
@@ -148,6 +151,7 @@ __global__ __launch_bounds__(kPfThreads) void chunk_prepare(const ChunkArgs g) {
   constexpr int C = kChunkTokens;
   __shared__ float sq[C][kMaxHeadDim], sk[C][kMaxHeadDim], sg[C][kMaxHeadDim];
   __shared__ __align__(16) float sa[C][C], sb[C][C];
+  __shared__ float step[C];
   const QmkHybridLayer& l = g.layer;
   const int dim = l.head_dim, n = l.v_dim, head = blockIdx.y, chunk = blockIdx.x, m0 = chunk * C, count = min(C, g.M - m0);
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -162,16 +166,17 @@ __global__ __launch_bounds__(kPfThreads) void chunk_prepare(const ChunkArgs g) {
       const T* x = static_cast<const T*>(g.raw) + ch;
       const float* old = l.shift + (static_cast<size_t>(g.slot) * 2 + g.flip) * (taps - 1) * W + ch;
       const float* weight = l.vec2 + ch;
-      auto input = [&](int at) {      // token at of the portion; tokens behind it are not used
-        return at >= 0 ? to_f32(x[static_cast<size_t>(min(at, g.M - 1)) * W]) : old[static_cast<size_t>(at + taps - 1) * W];
-      };
+      auto inside = [&](int at) { return to_f32(x[static_cast<size_t>(min(at, g.M - 1)) * W]); };      // tokens behind the portion are not used
+      auto input = [&](int at) { return at >= 0 ? inside(at) : old[static_cast<size_t>(at + taps - 1) * W]; };
       constexpr int kFew = 4;
       if (taps <= kFew) {
         float in[C + kFew - 1], w[kFew];
 #pragma unroll
         for (int j = 0; j < kFew; ++j) w[j] = j >= kFew - taps ? weight[static_cast<size_t>(j - kFew + taps) * W] : 0.f;
 #pragma unroll
-        for (int j = 0; j < C + kFew - 1; ++j) in[j] = j >= kFew - taps ? input(m0 - (kFew - 1) + j) : 0.f;
+        for (int j = 0; j < kFew - 1; ++j) in[j] = j >= kFew - taps ? input(m0 - (kFew - 1) + j) : 0.f;
+#pragma unroll
+        for (int j = 0; j < C; ++j) in[kFew - 1 + j] = inside(m0 + j);
 #pragma unroll
         for (int t = 0; t < C; ++t) {
           v[t] = 0.f;
@@ -204,6 +209,9 @@ __global__ __launch_bounds__(kPfThreads) void chunk_prepare(const ChunkArgs g) {
 #pragma unroll
     for (int t = 0; t < C; ++t) to[t][c] = t < count ? v[t] : 0.f;
   }
+  if constexpr (DELTA) {
+    if (tid < count) step[tid] = g.beta[static_cast<size_t>(m0 + tid) * g.beta_ld + head];
+  }
   for (int c = tid; c < dim; c += kPfThreads) {
     const float* row = g.decay + static_cast<size_t>(m0) * l.heads * dim + head * dim + c;
     float v[C];
@@ -230,8 +238,10 @@ __global__ __launch_bounds__(kPfThreads) void chunk_prepare(const ChunkArgs g) {
   }
 
   float* rec = g.chunks + (static_cast<size_t>(chunk) * l.heads + head) * chunk_floats(dim);
-  const int tiles = dim / 16;
-  float *rq = rec, *rk = rq + tiles * 256, *rd = rk + tiles * 256, *rg = rd + tiles * 256, *rb = rg + dim, *rt = rb + 256;
+  const int tiles = dim / 16, stored = chunk_tiles(dim);
+  float *rq = rec, *rk = rq + stored * 256, *rd = rk + stored * 256, *rg = rd + stored * 256, *rb = rg + stored * 16, *rt = rb + 256;
+  for (int i = tiles * 256 + tid; i < stored * 256; i += kPfThreads) rq[i] = rk[i] = rd[i] = 0.f;
+  if (tid >= dim && tid < stored * 16) rg[tid] = 0.f;
   if (tid < dim) {
     const int tile = tid >> 4, c = tid & 15;
     float cum = 1.f;
@@ -294,7 +304,7 @@ __global__ __launch_bounds__(kPfThreads) void chunk_prepare(const ChunkArgs g) {
         float acc = t == tid ? 1.f : 0.f;
 #pragma unroll
         for (int j = 0; j < t; ++j) acc = fmaf(-sa[t][j], col[j], acc);
-        col[t] = t < count ? acc * g.beta[static_cast<size_t>(m0 + t) * g.beta_ld + head] : 0.f;
+        col[t] = t < count ? acc * step[t] : 0.f;
         rt[((tid >> 2) * 16 + t) * 4 + (tid & 3)] = col[t];
       }
     }
@@ -315,21 +325,25 @@ __global__ __launch_bounds__(kPfThreads) void keep_inputs(const T* x, QmkHybridL
 }
 
 // One head and sixteen value columns a workgroup; a wave holds TILES tiles of sixteen key channels of the state as the
-// accumulators of the matrix instruction, which are also the second operand of the products that read it.  A wave's tiles
-// behind the last one are zeros and take part: with a branch around each tile's products this compiler has left out the wait
-// between a tile's last product and the first use of its result on the path that skips the next tile.
+// accumulators of the matrix instruction, which are also the second operand of the products that read it.  Tiles behind the
+// last one are zeros and take part: with a branch around each tile's products this compiler has left out the wait between a
+// tile's last product and the first use of its result on the path that skips the next tile.  Loads have no branches either,
+// so that kAhead chunks are in flight: a chunk, or token, behind the last one is the last one again, and its value is either
+// not used or multiplied by zero.
 template <int TILES, bool DELTA>
 __global__ __launch_bounds__(kChunkWaves * 64) void chunk_scan(const ChunkArgs g) {
   constexpr int kAhead = TILES <= 2 ? 4 : 2;      // chunks in flight
   __shared__ f32x4 px[2][kChunkWaves][64], po[2][kChunkWaves][64];
   const QmkHybridLayer& l = g.layer;
-  const int dim = l.head_dim, n = l.v_dim, head = blockIdx.x, v0 = blockIdx.y * 16, tiles = dim / 16;
+  const int dim = l.head_dim, n = l.v_dim, head = blockIdx.x, v0 = blockIdx.y * 16;
+  constexpr int tiles = TILES * kChunkWaves;
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), col = lane & 15, quad = lane >> 4;
-  const int tile0 = wave * TILES, mine = min(max(tiles - tile0, 0), TILES);
+  const int tile0 = wave * TILES, mine = min(max(dim / 16 - tile0, 0), TILES);
   const int chunks = (g.M + kChunkTokens - 1) / kChunkTokens;
   const size_t step = static_cast<size_t>(l.heads) * chunk_floats(dim);
   const float* rec = g.chunks + static_cast<size_t>(head) * chunk_floats(dim);
   float* state = l.state + (static_cast<size_t>(g.slot) * l.heads + head) * dim * n + v0 + col;
+  const float* values = g.values + g.value_at + head * n + v0 + col;
   f32x4 s[TILES];
 #pragma unroll
   for (int j = 0; j < TILES; ++j)
@@ -340,33 +354,27 @@ __global__ __launch_bounds__(kChunkWaves * 64) void chunk_scan(const ChunkArgs g
     f32x4 q[TILES], k[TILES], d[TILES], g[TILES], b, t, v;
   };
   auto fetch = [&](Fragments& f, int chunk) {
+    chunk = min(chunk, chunks - 1);
     const float* r = rec + chunk * step;
 #pragma unroll
     for (int j = 0; j < TILES; ++j) {
-      const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
-      f.q[j] = f.k[j] = f.d[j] = f.g[j] = zero;
-      if (j < mine) {
-        const int at = (tile0 + j) * 256 + lane * 4;
-        f.q[j] = read4(r + at);
-        if constexpr (DELTA) f.k[j] = read4(r + tiles * 256 + at);
-        f.d[j] = read4(r + tiles * 512 + at);
-        f.g[j] = read4(r + tiles * 768 + (tile0 + j) * 16 + quad * 4);
-      }
+      const int at = (tile0 + j) * 256 + lane * 4;
+      if constexpr (DELTA) f.k[j] = read4(r + tiles * 256 + at);
+      f.q[j] = read4(r + at);
+      f.d[j] = read4(r + tiles * 512 + at);
+      f.g[j] = read4(r + tiles * 768 + (tile0 + j) * 16 + quad * 4);
     }
     f.b = read4(r + tiles * 784 + lane * 4);
     if constexpr (DELTA) f.t = read4(r + tiles * 784 + 256 + lane * 4);
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int m = chunk * kChunkTokens + quad * 4 + i;
-      f.v[i] = m < g.M ? g.values[static_cast<size_t>(m) * g.value_ld + g.value_at + head * n + v0 + col] : 0.f;
-    }
+    for (int i = 0; i < 4; ++i) f.v[i] = values[static_cast<size_t>(min(chunk * kChunkTokens + quad * 4 + i, g.M - 1)) * g.value_ld];
   };
   auto product = [](f32x4 a, f32x4 b, f32x4 c) {
 #pragma unroll
     for (int i = 0; i < 4; ++i) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], b[i], c, 0, 0, 0);
     return c;
   };
-  auto advance = [&](Fragments& f, int chunk) {      // ... and the fragments' place is filled again
+  auto advance = [&](const Fragments& f, int chunk) {
     const int buf = chunk & 1;
     f32x4 x = {}, o = {};
     if constexpr (DELTA) {
@@ -396,17 +404,21 @@ __global__ __launch_bounds__(kChunkWaves * 64) void chunk_scan(const ChunkArgs g
         if (m < g.M) g.out[static_cast<size_t>(m) * l.heads * n + head * n + v0 + col] = o[i];
       }
     }
-    if (chunk + kAhead < chunks) fetch(f, chunk + kAhead);
   };
   Fragments f[kAhead];
 #pragma unroll
-  for (int a = 0; a < kAhead; ++a)
-    if (a < chunks) fetch(f[a], a);
-  for (int chunk = 0; chunk < chunks; chunk += kAhead) {
+  for (int a = 0; a < kAhead; ++a) fetch(f[a], a);
+  int chunk = 0;
+  for (; chunk + kAhead <= chunks; chunk += kAhead) {
 #pragma unroll
-    for (int a = 0; a < kAhead; ++a)
-      if (chunk + a < chunks) advance(f[a], chunk + a);
+    for (int a = 0; a < kAhead; ++a) {
+      advance(f[a], chunk + a);
+      fetch(f[a], chunk + a + kAhead);
+    }
   }
+#pragma unroll
+  for (int a = 0; a < kAhead - 1; ++a)
+    if (chunk + a < chunks) advance(f[a], chunk + a);
 #pragma unroll
   for (int j = 0; j < TILES; ++j)
     if (j < mine)
