@@ -620,7 +620,10 @@ __global__ __launch_bounds__(kPfThreads) void window_attention(const T* q, Keys<
   __shared__ __align__(16) T sk[kKeys][QT * 32 + kPadK];
   __shared__ __align__(16) T sv[VT * 16][kKeys + kPadV];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g = lane >> 4, col = lane & 15;
-  const int head = blockIdx.y, kv = head / keys.heads_per, q0 = (gridDim.x - 1 - blockIdx.x) * 64;      // the longest rows of keys first
+  // Later queries see more keys where no window ends.  Workgroups 256 apart share a CU: every other such run of heads takes
+  // its queries from the far end, so that a CU gets long and short ones.
+  const bool mirrored = (blockIdx.y * gridDim.x >> 8 & 1) == 0;
+  const int head = blockIdx.y, kv = head / keys.heads_per, q0 = (mirrored ? gridDim.x - 1 - blockIdx.x : blockIdx.x) * 64;
   const int dq = l.q_stride, steps = dq / 32, vt = l.v_dim / 16, width = l.rank + l.rot_dim;
   const int m = q0 + wave * 16 + col, pos = position + m;
   Frag<T> fq[QT];

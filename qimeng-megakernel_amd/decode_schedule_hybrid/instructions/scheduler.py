@@ -55,10 +55,26 @@ class HybridScheduler:
     max_positions: int = 1 << 30
 
     def parts(self, layer: int) -> int:
-        """Parts the visible keys of an attention are cut into."""
-        l = self.shape.entries[layer].shape
+        """Parts the visible keys of an attention are cut into; where other branches run in the same stage, no more than fit
+        beside them (but at least eight)."""
+        entry = self.shape.entries[layer]
+        l, most = entry.shape, MAX_PARTS
         reach = min(l.window, self.max_positions) if l.type == "latent_attention" else self.max_positions
-        return max(1, min(MAX_PARTS, _ceil_div(reach, KEYS_PER_PART)))
+        if entry.branches > 1:
+            beside = [e.shape for e in self.shape.entries[layer - entry.branch : layer - entry.branch + entry.branches] if e.type != "attention"]
+            busy = sum(b.heads * _ceil_div(b.v_s, STATE_COLUMNS) for b in beside) + (self.gate_instructions if any(b.gate_rank for b in beside) else 0)
+            most = min(MAX_PARTS, max(8, (self.queues - busy) // len(self.attention_groups(l))))
+        return max(1, min(most, _ceil_div(reach, KEYS_PER_PART)))
+
+    @property
+    def gate_instructions(self) -> int:
+        """Instructions the rows of a low-rank gate are cut into."""
+        return max(1, self.queues // 8)
+
+    @staticmethod
+    def attention_groups(l: Any) -> list[tuple[int, int]]:
+        """(key head and sixteen of its heads, value columns) of the instructions that make one part of an attention."""
+        return [(g, c) for g in range(l.kv_heads * _ceil_div(l.heads // l.kv_heads, 16)) for c in range(_ceil_div(l.v_s, ATTEND_COLUMNS))]
 
     def max_parts(self) -> int:
         return max([self.parts(i) for i, e in enumerate(self.shape.entries) if e.type in ("latent_attention", "attention")], default=1)
@@ -109,26 +125,25 @@ class HybridScheduler:
         stages[0][0].extra = 1
         steps: list[D.StageInstruction] = []
         merges: list[D.StageInstruction] = []
-        gates: list[tuple[int, Any]] = []
+        attend: list[D.StageInstruction] = []
         early: list[tuple[int, Any]] = []
         late: list[tuple[int, Any]] = []
         for i, l in branches.items():
             out = (width, lambda a, n, i=i: D.OutProject_Streams(i, 0, a, n))
             if l.type == "attention":
-                parts, blocks = self.parts(i), _ceil_div(l.heads // l.kv_heads, 16)
-                steps += [D.AttendSplitKV(i, g, part, parts, extra=c) for part in range(parts) for g in range(l.kv_heads * blocks)
-                          for c in range(_ceil_div(l.v_s, ATTEND_COLUMNS))]
+                parts = self.parts(i)
+                attend += [D.AttendSplitKV(i, g, part, parts, extra=c) for part in range(parts) for g, c in self.attention_groups(l)]
                 merges += [D.AttendMerge(i, h, 0, parts) for h in range(l.heads)]
                 late.append(out)
             else:
-                steps = [D.GatedStateStep(i, h, a, min(STATE_COLUMNS, l.v_s - a)) for h in range(l.heads) for a in range(0, l.v_s, STATE_COLUMNS)] + steps
+                steps += [D.GatedStateStep(i, h, a, min(STATE_COLUMNS, l.v_s - a)) for h in range(l.heads) for a in range(0, l.v_s, STATE_COLUMNS)]
                 if l.gate_rank:
-                    gates.append((l.mix_width, lambda a, n, i=i: D.OutputGate(i, 0, a, n)))
+                    steps += [D.OutputGate(i, 0, a, n) for _, a, n in cut([(0, l.mix_width)], self.gate_instructions)]
                 early.append(out)
         if merges:
-            stages += [steps + self._spread(gates, len(steps)), merges + self._spread(early + down, len(merges)), self._spread(late)]
+            stages += [steps + attend, merges + self._spread(early + down, len(merges)), self._spread(late)]
         else:
-            stages += [steps + self._spread(gates + down, len(steps)), self._spread(early)]
+            stages += [steps + self._spread(down, len(steps)), self._spread(early)]
         return stages
 
     def stages(self) -> list[list[D.StageInstruction]]:
