@@ -44,6 +44,8 @@ constexpr int kMaxRank = 512;
 constexpr int kMaxHeadDim = 256;              // wkv, gla, delta
 constexpr int kStateColumns = 64;             // value columns of one OP_STATE_STEP
 constexpr int kStateRows = 32;                // key rows of the state one of its threads holds: 256 rows / (512 / 64) threads a column
+constexpr int kStateBatch = 8;                // ... taken together, without branches: rows behind the last one count with weights of zero
+constexpr int kStateVector = kMaxHeadDim + kStateBatch * kThreads / 16;   // places of q, k and the decays in LDS, zeros behind head_dim
 constexpr int kMaxParts = 64;
 constexpr int kDepth = 8;                     // weight rows a wave keeps in flight and reduces together
 constexpr int kAhead = 2;                     // quads of a vector a thread holds in registers (4096 elements a workgroup)
@@ -718,10 +720,16 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
     const int n = o.count, groups = kThreads / n, e = tid % n, group = tid / n;
     state = l.state + (static_cast<size_t>(p.slot) * l.heads + o.sub) * l.head_dim * l.v_dim + o.start + e;
 #pragma unroll
-    for (int j = 0; j < kStateRows; ++j) {
-      const int i = group + j * groups;
-      held[j] = group < groups && i < l.head_dim ? state[static_cast<size_t>(i) * l.v_dim] : 0.f;
+    for (int j0 = 0; j0 < kStateRows; j0 += kStateBatch) {
+      if (j0 * groups < l.head_dim) {
+#pragma unroll
+        for (int j = j0; j < j0 + kStateBatch; ++j) held[j] = state[static_cast<size_t>(min(group + j * groups, l.head_dim - 1)) * l.v_dim];
+      }
     }
+    static_assert(3 * kStateVector + kStateColumns <= 3072 && kStateVector <= 2 * kThreads, "q, k, decays and values in aux");
+#pragma unroll
+    for (int i = 0; i < 3; ++i)
+      for (int at = l.head_dim + tid; at < kStateVector; at += kThreads) s.aux[i * kStateVector + at] = 0.f;
     if (mine) a[0] = l.mid_b[o.sub * l.head_dim + tid];
   } else if (op == OP_OUT_PROJECT && !plain) {
     // Eight lanes per row, one per stream: all streams of the row, the stream's column of the mix, its output weight and
@@ -814,7 +822,7 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
         q = ld_shared_f32(proj + kv * dim + tid);
         k = ld_shared_f32(proj + keys + kv * dim + tid);
       }
-      if (tid < o.count) s.aux[2 * kMaxHeadDim + tid] = ld_shared_f32(proj + 2 * keys + o.sub * n + o.start + tid);
+      if (tid < o.count) s.aux[3 * kStateVector + tid] = ld_shared_f32(proj + 2 * keys + o.sub * n + o.start + tid);
       from = proj + 2 * keys + l.heads * n * (delta ? 1 : 2);
       if (delta) a[3] = ld_shared_f32(from + l.rank + l.gate_rank + o.sub);      // beta
       if (!delta) q *= l.q_scale;                       // (the projection is left unscaled)
@@ -829,7 +837,7 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
       a[4] = dots[2];
       if (tid < dim) {
         s.aux[tid] = q;
-        s.aux[kMaxHeadDim + tid] = k;
+        s.aux[kStateVector + tid] = k;
       }
     } else if (plain && op == OP_GATE) {
       from = p.proj + l.proj_at + conv_channels(l) + l.rank;
@@ -1004,20 +1012,23 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
     // o = (decay S)^T q + (q . k) u.  Without the delta rule u = v.
     const bool delta = type == QMK_MIXER_DELTA;
     const int n = o.count, dim = l.head_dim, groups = kThreads / n, e = tid % n, group = tid / n;
-    float *q = s.aux, *k = q + kMaxHeadDim, *v = k + kMaxHeadDim, *w = v + kMaxHeadDim;
+    float *q = s.aux, *k = q + kStateVector, *w = k + kStateVector, *v = w + kStateVector;
     if (mine) w[tid] = delta ? delta_decay(l, o.sub, t + a[0]) : gla_decay(l, t + a[0]);
     __syncthreads();
     float ak = 0.f, aq = 0.f;
-    if (group < groups) {
 #pragma unroll
-      for (int j = 0; j < kStateRows; ++j) {
-        const int i = group + j * groups;
-        if (i < dim) {
+    for (int j0 = 0; j0 < kStateRows; j0 += kStateBatch) {
+      if (j0 * groups < dim) {
+#pragma unroll
+        for (int j = j0; j < j0 + kStateBatch; ++j) {
+          const int i = group + j * groups;
           held[j] *= w[i];
           ak = fmaf(k[i], held[j], ak);
           aq = fmaf(q[i], held[j], aq);
         }
       }
+    }
+    if (group < groups) {
       s.xs[group * n + e] = ak;
       s.xs[(groups + group) * n + e] = aq;
     }
@@ -1031,9 +1042,15 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
     const float u = delta ? a[3] * (v[e] - ak) : v[e];
     if (group < groups) {
 #pragma unroll
-      for (int j = 0; j < kStateRows; ++j) {
-        const int i = group + j * groups;
-        if (i < dim) state[static_cast<size_t>(i) * l.v_dim] = fmaf(k[i], u, held[j]);
+      for (int j0 = 0; j0 < kStateRows; j0 += kStateBatch) {
+        if (j0 * groups < dim) {
+#pragma unroll
+          for (int j = j0; j < j0 + kStateBatch; ++j) {
+            const int i = group + j * groups;
+            const float now = fmaf(k[i], u, held[j]);
+            if (i < dim) state[static_cast<size_t>(i) * l.v_dim] = now;
+          }
+        }
       }
     }
     if (tid < n) st_shared_f32(p.mix + l.mix_at + o.sub * l.v_dim + o.start + tid, fmaf(a[4], u, aq));
