@@ -1040,6 +1040,9 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
       aq += s.xs[(groups + i) * n + e];
     }
     const float u = delta ? a[3] * (v[e] - ak) : v[e];
+    if (tid < n) st_shared_f32(p.mix + l.mix_at + o.sub * l.v_dim + o.start + tid, fmaf(a[4], u, aq));
+    stamp(p, s, 3);
+    arrive_stage(p, o);      // nobody else reads the state in this launch: its stores need no acknowledgement before the arrival
     if (group < groups) {
 #pragma unroll
       for (int j0 = 0; j0 < kStateRows; j0 += kStateBatch) {
@@ -1053,7 +1056,7 @@ __device__ __forceinline__ bool op_rows(const DecodeParams& p, Smem& s, const Op
         }
       }
     }
-    if (tid < n) st_shared_f32(p.mix + l.mix_at + o.sub * l.v_dim + o.start + tid, fmaf(a[4], u, aq));
+    return true;
   } else if (plain && op == OP_GATE) {
     if (mine) st_shared_f32(p.proj + l.proj_at + l.in_rows + row, sigmoid(t));
   } else {   // OP_LM_HEAD
