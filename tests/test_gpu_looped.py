@@ -24,7 +24,7 @@ BOTH = pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16], ids=["f
 #: sizes off and on the storage multiples, grouped heads everywhere, loops at either end, with and without feed-forwards
 SHAPES = {
     "odd": synthetic.looped_shape("pgp", width=52, vocab=77, ff={"p": 36}, loop=(1, 3, 2), logit_scale=0.7, logit_softcap=4.0, heads=6, kv_heads=2, dim=20,
-                                  v_dim=12, rot_dim=10, rope_base=50.0, rope_scaling=(3.0, 40.0, 6.0, 0.7), scale=0.31, delta_heads=6, delta_kv_heads=3,
+                                  v_dim=12, rot_dim=10, rope_base=50.0, rope_scaling=(3.0, 40.0, 2.0, 0.7), scale=0.31, delta_heads=6, delta_kv_heads=3,
                                   delta_dim=12, delta_v_dim=20, taps=4, delta_rank=7, gate_rank=5, gla_heads=3, gla_dim=20, gla_v_dim=28, gla_rank=9, tau=5.0),
     "from_the_start": synthetic.looped_shape("gp", width=64, vocab=130, ff={"g": 48, "p": 16}, loop=(0, 2, 3), heads=2, kv_heads=2, dim=32, v_dim=16, rot_dim=32,
                                              delta_heads=2, delta_kv_heads=1, delta_dim=16, delta_v_dim=16, taps=1, delta_rank=16, gate_rank=16, gla_heads=1,
