@@ -324,13 +324,13 @@ inline size_t values_cap(const QmkHybridArgs* a) { return (static_cast<size_t>(a
 
 template <class T>
 struct PlainBuffers {
-  float *x, *branch, *qkv, *decay, *beta, *o, *chunks;
+  float *x, *branch, *qkv, *values, *decay, *beta, *o, *chunks;
   T *h, *q, *low, *gate, *mix, *vt;
 };
 template <class T>
 size_t plain_buffers(const QmkHybridArgs* a, void* base, PlainBuffers<T>* b) {
   const size_t P = a->portion_rows, D = a->width, chunks_of = (P + kChunkTokens - 1) / kChunkTokens;
-  size_t h = P * D, branch = 0, qkv = 0, decay = 0, beta = 0, o = 0, chunks = 0, q = 0, low = 0, gate = 0, mix = 0, vt = 0;
+  size_t h = P * D, branch = 0, qkv = 0, values = 0, decay = 0, beta = 0, o = 0, chunks = 0, q = 0, low = 0, gate = 0, mix = 0, vt = 0;
   for (int i = 0; i < a->num_layers; ++i) {
     const QmkHybridLayer& l = a->layers[i];
     if (l.type == QMK_ENTRY_JOIN) h = std::max(h, 2 * P * D);
@@ -348,8 +348,8 @@ size_t plain_buffers(const QmkHybridArgs* a, void* base, PlainBuffers<T>* b) {
     low = std::max(low, P * (l.rank + l.gate_rank));
     chunks = std::max(chunks, chunks_of * l.heads * chunk_floats(l.head_dim));
     if (l.type == QMK_MIXER_DELTA) {
-      q = std::max(q, P * conv_channels(l));
-      qkv = std::max(qkv, P * l.mix_width);
+      qkv = std::max(qkv, P * conv_channels(l));
+      values = std::max(values, P * l.mix_width);
       beta = std::max(beta, P * ((l.heads + 15) / 16 * 16));
     } else {
       qkv = std::max(qkv, P * (2 * l.heads * l.head_dim + l.mix_width));
@@ -361,6 +361,7 @@ size_t plain_buffers(const QmkHybridArgs* a, void* base, PlainBuffers<T>* b) {
   b->x = c.take<float>(P * D);
   b->branch = c.take<float>(branch);
   b->qkv = c.take<float>(qkv);
+  b->values = c.take<float>(values);
   b->decay = c.take<float>(decay);
   b->beta = c.take<float>(beta);
   b->o = c.take<float>(o);
@@ -553,11 +554,11 @@ int prefill(const QmkHybridArgs* a) {
 }
 
 // The recurrence of a gla or delta entry over the portion, from its projections to what its output projection reads.
-template <class T, bool DELTA>
+template <bool DELTA>
 void run_chunks(const QmkHybridArgs* a, const ChunkArgs& g, hipStream_t st) {
   const QmkHybridLayer& l = g.layer;
   const int chunks = (g.M + kChunkTokens - 1) / kChunkTokens, tiles = wave_tiles(l.head_dim);
-  hipLaunchKernelGGL((chunk_prepare<T, DELTA>), dim3(chunks, l.heads), dim3(kPfThreads), 0, st, g);
+  hipLaunchKernelGGL(chunk_prepare<DELTA>, dim3(chunks, l.heads), dim3(kPfThreads), 0, st, g);
   const dim3 grid(l.heads, l.v_dim / 16), block(kChunkWaves * 64);
   if (tiles == 1) hipLaunchKernelGGL((chunk_scan<1, DELTA>), grid, block, 0, st, g);
   else if (tiles == 2) hipLaunchKernelGGL((chunk_scan<2, DELTA>), grid, block, 0, st, g);
@@ -630,7 +631,7 @@ int prefill_plain(const QmkHybridArgs* a) {
       if (l.type == QMK_MIXER_DELTA) {
         const int channels = conv_channels(l), ranks = l.rank + l.gate_rank, beta_ld = (l.heads + 15) / 16 * 16;
         GemmArgs g = gemm_args(b.h, l.in_w, l.in_rows, D, l, EPI_DELTA_IN);
-        g.out = b.q; g.out2 = b.low; g.f0 = b.beta; g.ldo = beta_ld;
+        g.f1 = b.qkv; g.out2 = b.low; g.f0 = b.beta; g.ldo = beta_ld;
         launch_gemm<T, u16, T>(g, st);
         const int keys = l.heads * l.head_dim;
         GemmArgs e = gemm_args(b.low, l.mid_w, keys, l.rank, l, EPI_DELTA_DECAY);
@@ -639,10 +640,10 @@ int prefill_plain(const QmkHybridArgs* a) {
         GemmArgs f = gemm_args(b.low + l.rank, l.gate_w, W, l.gate_rank, l, EPI_SIGMOID);
         f.lda = ranks; f.out = b.gate; f.ldo = W;
         launch_gemm<T, u16, T>(f, st);
-        c.raw = b.q; c.beta = b.beta; c.beta_ld = beta_ld; c.values = b.qkv; c.value_ld = W;
-        run_chunks<T, true>(a, c, st);
+        c.qkv = b.qkv; c.beta = b.beta; c.beta_ld = beta_ld; c.values = b.values; c.value_ld = W;
+        run_chunks<true>(a, c, st);
         if (l.taps > 1)
-          hipLaunchKernelGGL(keep_inputs<T>, dim3((channels + kPfThreads - 1) / kPfThreads), block, 0, st, b.q, l, channels, a->slot, a->flip, M);
+          hipLaunchKernelGGL(keep_inputs, dim3((channels + kPfThreads - 1) / kPfThreads), block, 0, st, b.qkv, l, channels, a->slot, a->flip, M);
       } else {
         const int keys = l.heads * l.head_dim;
         GemmArgs g = gemm_args(b.h, l.in_w, l.in_rows, D, l, EPI_GLA_IN);
@@ -652,7 +653,7 @@ int prefill_plain(const QmkHybridArgs* a) {
         e.f0 = b.decay; e.ldo = keys;
         launch_gemm<T, u16, T>(e, st);
         c.qkv = b.qkv; c.values = b.qkv; c.value_ld = 2 * keys + W; c.value_at = 2 * keys;
-        run_chunks<T, false>(a, c, st);
+        run_chunks<false>(a, c, st);
       }
       hipLaunchKernelGGL(state_out<T>, dim3((M * l.heads + 3) / 4), block, 0, st, b.o, b.gate, l, M, a->eps, b.mix);
     }

@@ -135,8 +135,7 @@ __host__ __device__ constexpr int chunk_floats(int head_dim) { return chunk_tile
 
 struct ChunkArgs {
   QmkHybridLayer layer;
-  const void* raw;       // delta: T [M][channels] projections of q, k, v ahead of the convolution
-  const float* qkv;      // gla: [M][q, k, v]
+  const float* qkv;      // [M][q, k, v]; delta: ahead of the convolution
   const float* decay;    // [M][heads * head_dim]
   const float* beta;     // delta: [M][beta_ld]
   float* chunks;         // [chunk][head][chunk_floats]
@@ -146,7 +145,7 @@ struct ChunkArgs {
 };
 
 // One workgroup per (chunk, head).  delta: convolution, silu and unit norm of the head's q and k, convolution and silu of its v.
-template <class T, bool DELTA>
+template <bool DELTA>
 __global__ __launch_bounds__(kPfThreads) void chunk_prepare(const ChunkArgs g) {
   constexpr int C = kChunkTokens;
   __shared__ float sq[C][kMaxHeadDim], sk[C][kMaxHeadDim], sg[C][kMaxHeadDim];
@@ -163,10 +162,10 @@ __global__ __launch_bounds__(kPfThreads) void chunk_prepare(const ChunkArgs g) {
     float v[C];
     if constexpr (DELTA) {
       const int W = conv_channels(l), taps = l.taps, ch = part == 0 ? kv * dim + c : part == 1 ? keys + kv * dim + c : 2 * keys + head * n + c;
-      const T* x = static_cast<const T*>(g.raw) + ch;
+      const float* x = g.qkv + ch;
       const float* old = l.shift + (static_cast<size_t>(g.slot) * 2 + g.flip) * (taps - 1) * W + ch;
       const float* weight = l.vec2 + ch;
-      auto inside = [&](int at) { return to_f32(x[static_cast<size_t>(min(at, g.M - 1)) * W]); };      // tokens behind the portion are not used
+      auto inside = [&](int at) { return x[static_cast<size_t>(min(at, g.M - 1)) * W]; };      // tokens behind the portion are not used
       auto input = [&](int at) { return at >= 0 ? inside(at) : old[static_cast<size_t>(at + taps - 1) * W]; };
       constexpr int kFew = 4;
       if (taps <= kFew) {
@@ -312,15 +311,14 @@ __global__ __launch_bounds__(kPfThreads) void chunk_prepare(const ChunkArgs g) {
 }
 
 // The convolution's last inputs of a portion, for the next one.
-template <class T>
-__global__ __launch_bounds__(kPfThreads) void keep_inputs(const T* x, QmkHybridLayer l, int W, int slot, int flip, int M) {
+__global__ __launch_bounds__(kPfThreads) void keep_inputs(const float* x, QmkHybridLayer l, int W, int slot, int flip, int M) {
   const int c = blockIdx.x * kPfThreads + threadIdx.x, n = l.taps - 1;
   if (c >= W) return;
   const float* old = l.shift + (static_cast<size_t>(slot) * 2 + flip) * n * W;
   float* now = l.shift + (static_cast<size_t>(slot) * 2 + 1 - flip) * n * W;
   for (int j = 0; j < n; ++j) {
     const int t = M - n + j;
-    now[static_cast<size_t>(j) * W + c] = t >= 0 ? to_f32(x[static_cast<size_t>(t) * W + c]) : old[static_cast<size_t>(t + n) * W + c];
+    now[static_cast<size_t>(j) * W + c] = t >= 0 ? x[static_cast<size_t>(t) * W + c] : old[static_cast<size_t>(t + n) * W + c];
   }
 }
 

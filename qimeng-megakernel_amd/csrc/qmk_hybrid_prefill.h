@@ -25,7 +25,7 @@ enum : int {
   EPI_CAPPED_LOGITS,    // logits times a constant, softly capped
   EPI_ADD,              // onto the fp32 residual
   EPI_ATTENTION_IN,     // rotation of q and k, k and v into the cache, sigmoid of the gate
-  EPI_DELTA_IN,         // raw q, k, v; raw ranks; sigmoid of the step sizes
+  EPI_DELTA_IN,         // q, k, v fp32; raw ranks; sigmoid of the step sizes
   EPI_DELTA_DECAY,
   EPI_SIGMOID,
   EPI_GLA_IN,           // q, k, v fp32; silu gate; raw rank
@@ -214,7 +214,7 @@ __device__ __forceinline__ void epilogue(const GemmArgs& g, int group, int m, in
     case EPI_DELTA_IN: {
       const int channels = conv_channels(l), ranks = l.rank + l.gate_rank;
       if (n < channels) {
-        store4(static_cast<T*>(g.out) + static_cast<size_t>(m) * channels + n, v);
+        store4(g.f1 + static_cast<size_t>(m) * channels + n, v);
       } else if (n < channels + ranks) {
         store4(static_cast<T*>(g.out2) + static_cast<size_t>(m) * ranks + n - channels, v);
       } else {
