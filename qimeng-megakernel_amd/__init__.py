@@ -11,7 +11,7 @@ Layout:
   instruction.py    instruction wire format
   synthetic.py      seeded random-init weights and Globals allocation (no checkpoint needed)
   decode_schedule_hybrid/, decode_hybrid.py
-                    the hybrid route (Lusupel): configuration, checkpoint loading, per-slot states, scheduler, launcher;
+                    the hybrid route (Lusupel, Givopel): configuration, checkpoint loading, per-slot states, scheduler, launcher;
                     step function and greedy loop
   registry.py       model names and config.json architectures -> route
   decode.py         prefill-by-decode and the greedy step loop with the reference's timing

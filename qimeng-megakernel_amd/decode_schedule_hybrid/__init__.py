@@ -1,5 +1,6 @@
 """Route package of hybrid decoders: per-layer mixers (gated linear recurrence, wkv time mixing, latent attention) on a
-hyper-connected residual stream.  Exports the names every route package exports (``decode_schedule/__init__.py``)."""
+hyper-connected residual stream, or (gated linear attention, softmax attention beside a gated delta rule) on a plain residual
+that a stretch of layers may run over several times.  Exports the names every route package exports (``decode_schedule/__init__.py``)."""
 from __future__ import annotations
 
 import importlib

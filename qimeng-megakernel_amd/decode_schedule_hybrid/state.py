@@ -1,7 +1,7 @@
 """Requests and the slots that hold their state.
 
-A slot is one row of every layer's state: cache rows of the latent attention, recurrent states in fp32, the last inputs
-of a convolution and the previous token's input.  ``RequestTable`` hands slots out, clears what a new request must find
+A slot is one row of every state: cache rows of an attention, recurrent states in fp32, the last inputs of a convolution
+and the previous token's input; a layer that runs in several passes has a state per pass.  ``RequestTable`` hands slots out, clears what a new request must find
 cleared, and keeps what the host knows of a request: its position and which copy of the two-copy inputs is current.
 """
 from __future__ import annotations
